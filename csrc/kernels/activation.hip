@@ -276,3 +276,66 @@ EIA_API int eia_sigmoid_gate(const void* a, long lda, long a_sh, int V, const vo
                        V, (const float*)g, ldg, (float*)out, ldo, rows, N, vec);
   EIA_LAUNCH_CHECK();
 }
+
+// ---------------------------------------------------------------------------------------------
+// Per-layer token input: out[t, c] = act(u[t, c]) * table[ids[t], col0 + c] for c < N, zero for
+// N <= c < NP (the pad columns of the product that follows).  u is a stored row (type T) or the
+// fp32 split-K partials [sk, rows, ldp] of the GEMM that produced it; fp32 inside.
+template <typename T, int KIND>
+__global__ void __launch_bounds__(256)
+act_mul_embed_kernel(const T* __restrict__ u, long ldu, const float* __restrict__ part, int sk,
+                     long ldp, const int* __restrict__ ids, const T* __restrict__ table, long ldt,
+                     int col0, int vocab, T* __restrict__ out, int rows, int N, int NP) {
+  const long idx = (long)blockIdx.x * 256 + threadIdx.x;
+  if (idx >= (long)rows * NP) return;
+  const int row = idx / NP, c = idx % NP;
+  float o = 0.f;
+  if (c < N) {
+    float v = 0.f;
+    if (u) {
+      v = ld_f32<T>(u + (long)row * ldu, c);
+    } else {
+      const float* p = part + (long)row * ldp + c;
+#pragma unroll 4
+      for (int z = 0; z < sk; ++z) v += p[(long)z * rows * ldp];
+    }
+    const int tok = min(max(ids[row], 0), vocab - 1);
+    o = act_f<KIND>(v) * ld_f32<T>(table + (long)tok * ldt, col0 + c);
+  }
+  st_f32<T>(out, idx, o);
+}
+
+EIA_API int eia_act_mul_embed(const void* u, long ldu, const float* part, int sk, long ldp,
+                              const int* ids, const void* table, long ldt, int col0, int vocab,
+                              void* out, int rows, int N, int NP, int kind, int is_bf16,
+                              hipStream_t st) {
+  if (rows < 0 || N < 1 || NP < N || vocab < 1 || col0 < 0 || col0 + N > ldt || !ids || !table ||
+      !out || (u == nullptr) == (part == nullptr) || (part && (sk < 1 || ldp < N)))
+    return EIA_BAD_SHAPE;
+  if (kind != ACT_SILU && kind != ACT_GELU_TANH) return EIA_UNSUPPORTED;
+  if (rows == 0) return EIA_OK;
+  const dim3 grid((unsigned)(((long)rows * NP + 255) / 256));
+#define AME(TT, K)                                                                              \
+  hipLaunchKernelGGL((act_mul_embed_kernel<TT, K>), grid, dim3(256), 0, st, (const TT*)u, ldu,  \
+                     part, sk, ldp, ids, (const TT*)table, ldt, col0, vocab, (TT*)out, rows, N, NP)
+  if (is_bf16) {
+    if (kind == ACT_SILU) AME(bf16_t, ACT_SILU); else AME(bf16_t, ACT_GELU_TANH);
+  } else {
+    if (kind == ACT_SILU) AME(float, ACT_SILU); else AME(float, ACT_GELU_TANH);
+  }
+#undef AME
+  EIA_LAUNCH_CHECK();
+}
+
+// x <- cap * tanh(x / cap) over fp32 values (logit soft cap), in place.
+__global__ void __launch_bounds__(256) softcap_kernel(float* __restrict__ x, long n, float cap) {
+  for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n; i += (long)gridDim.x * 256)
+    x[i] = cap * tanhf(x[i] / cap);
+}
+
+EIA_API int eia_softcap(float* x, long n, float cap, hipStream_t st) {
+  if (n < 0 || !x || !(cap > 0.f)) return EIA_BAD_SHAPE;
+  if (n == 0) return EIA_OK;
+  hipLaunchKernelGGL(softcap_kernel, dim3(grid_for((n + 3) / 4)), dim3(256), 0, st, x, n, cap);
+  EIA_LAUNCH_CHECK();
+}

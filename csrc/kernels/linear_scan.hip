@@ -1,5 +1,6 @@
-// Linear-attention recurrences with ONE decay number per head and token on per-sequence state
-// slots: a matrix state S [dk, dv] per head that every token scales and adds an outer product to,
+// Linear-attention recurrences with one decay number per head and token (modes 0, 1) or per key
+// channel and token (mode 2) on per-sequence state slots: a matrix state S [dk, dv] per head that
+// every token scales and adds an outer product to,
 //
 //   S_t = a_t S_(t-1) + b_t k_t v_t^T,      o_t = S_t^T q_t        (the token sees itself)
 //
@@ -10,14 +11,17 @@
 //     m_t = max(f + m_(t-1), i),
 //     a_t = exp(f + m_(t-1) - m_t),  b_t = exp(i - m_t),  n_t = a_t n_(t-1) + b_t k_t,
 //     o_t <- o_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6);       m starts at 0, S and n at zero.
-// Both: q and k may be rotated by the token's position on their first rot_dims entries (pairs
+// mode 2 (a decay per key channel, "gated linear attention"): the row holds a low-rank branch of
+//   R columns; z = A2 lo + bias per channel (fp32), a_t = sigmoid(z)^(1/tau) = exp(logsigmoid(z) /
+//   tau) scales the state's ROWS (row i belongs to key channel i), b_t = 1.
+// All: q and k may be rotated by the token's position on their first rot_dims entries (pairs
 // (i, i + rot_dims/2) or (2i, 2i+1)), then scaled (qscale, kscale); each head's o is divided by
 // its root mean square, multiplied by an optional weight and by silu or sigmoid of the gate
 // columns, and by out_scale.
 //
 // q, k, v, the gate and the gate pre-activations are column ranges of one fused projection row
 // per token (type T: bf16 or float).  Decays, gates, exponentials, the state, the normaliser and
-// the head norm are fp32.  A sequence whose first row of the step is position 0 starts from the
+// the head norm are fp32, as is mode 2's last decay product.  A sequence whose first row of the step is position 0 starts from the
 // initial state whatever its slot held, so slots are reused without clearing.
 // Batch layout: sequence s owns rows [cu[s], cu[s+1]) (cu == nullptr: row s).
 #include "eia_common.h"
@@ -34,9 +38,22 @@ struct ScanArgs {
   void* y; long ldy;                        // [rows, >= H * Dv]
   float eps;
   int H, D, Dv, mode, gate_act;
+  // mode 2: low-rank columns, A2 transposed [R, H * D], bias [H * D], 1 / tau
+  int lo_off, R; const float* a2t; const float* a2b; float inv_tau;
+  int norm_h;                               // columns of norm_w per head: 0: [Dv] shared by heads
 };
 
 EIA_DEV float ls_logsigmoid(float z) { return -(log1pf(expf(-fabsf(z))) + fmaxf(-z, 0.f)); }
+
+// log decay of channel j of head h for one row (mode 2)
+template <typename T>
+EIA_DEV float ls_chan_log(const ScanArgs& a, const T* xr, int h, int j) {
+  const float* w = a.a2t + (long)h * a.D + j;
+  float z = a.a2b ? a.a2b[(long)h * a.D + j] : 0.f;
+#pragma unroll 8
+  for (int r = 0; r < a.R; ++r) z += ld_f32<T>(xr, a.lo_off + r) * w[(long)r * a.H * a.D];
+  return ls_logsigmoid(z) * a.inv_tau;
+}
 
 // One workgroup per (sequence, head), 4 x max(64, DMAX) threads: thread (qt, j) owns rows
 // [qt DMAX/4, (qt+1) DMAX/4) of column j of S in registers and walks the sequence's tokens in
@@ -44,9 +61,9 @@ EIA_DEV float ls_logsigmoid(float z) { return -(log1pf(expf(-fabsf(z))) + fmaxf(
 // to LDS, the gate recurrence of the chunk runs (its transcendentals in parallel over the
 // tokens, the running maximum serially in one thread), then the state recurrence runs TC steps on
 // LDS broadcasts leaving four partial outputs per token and column, which are summed, divided,
-// normed and gated.  NRM: the normaliser n rides along (every thread of a quarter keeps the
+// normed and gated.  CH: a decay per key channel (mode 2), staged beside k.  NRM: the normaliser n rides along (every thread of a quarter keeps the
 // quarter's rows of n; column 0 reports n . q).
-template <typename T, int DMAX, bool NRM>
+template <typename T, int DMAX, bool NRM, bool CH>
 __global__ void __launch_bounds__(4 * (DMAX < 64 ? 64 : DMAX))
 linear_scan_kernel(ScanArgs a) {
   constexpr int DP = DMAX < 64 ? 64 : DMAX;          // threads per quarter
@@ -55,6 +72,7 @@ linear_scan_kernel(ScanArgs a) {
   constexpr int NWV = DP / 64;
   __shared__ __align__(16) float sq[TC][DMAX], sk[TC][DMAX];
   __shared__ float sv[TC][DMAX], sg[TC][DMAX], po[TC][4][DP];
+  __shared__ __align__(16) float sal[CH ? TC : 1][CH ? DMAX : 1];
   __shared__ float sa[TC], sb[TC], se[TC], gi[TC], gf[TC], pn[TC][4];
   __shared__ float red[4][NWV];
   __shared__ float m_run;
@@ -81,7 +99,7 @@ linear_scan_kernel(ScanArgs a) {
   const T* X = static_cast<const T*>(a.x);
   const T* NW = static_cast<const T*>(a.norm_w);
   T* Y = static_cast<T*>(a.y);
-  const float nw = (NW && col) ? ld_f32<T>(NW, (long)h * Dv + j) : 1.f;
+  const float nw = (NW && col) ? ld_f32<T>(NW, (long)h * a.norm_h + j) : 1.f;
   const float inv_dv = 1.0f / (float)Dv;
   // rotation of channel j: partner channel, the pair's frequency and the sign of the cross term
   const int hd = a.rot_dims >> 1;
@@ -125,6 +143,7 @@ linear_scan_kernel(ScanArgs a) {
           }
           sq[t][j] = q;
           sk[t][j] = k;
+          if constexpr (CH) sal[t][j] = chan ? expf(ls_chan_log<T>(a, xr, h, j)) : 1.f;
           sv[t][j] = v;
           sg[t][j] = g;
         }
@@ -164,7 +183,7 @@ linear_scan_kernel(ScanArgs a) {
 #pragma unroll
       for (int i = 0; i < DQ; ++i) {
         const float bk = bt * sk[t][i0 + i];
-        S[i] = at * S[i] + bk * v;
+        S[i] = (CH ? sal[t][i0 + i] : at) * S[i] + bk * v;
         o += sq[t][i0 + i] * S[i];
         if constexpr (NRM) {
           Nn[i] = at * Nn[i] + bk;
@@ -231,9 +250,11 @@ EIA_API int eia_linear_scan(const void* x, long ld, int q_off, int k_off, int v_
                             float out_scale, const void* norm_w, float* S, float* N, float* M,
                             const int* slots, const int* cu, const int* positions,
                             const int* seq_lens, void* y, long ldy, float eps, int nseq, int H,
-                            int D, int Dv, int mode, int gate_act, int is_bf16, hipStream_t st) {
+                            int D, int Dv, int mode, int gate_act, int lo_off, int R,
+                            const float* a2t, const float* a2b, float inv_tau, int norm_h,
+                            int is_bf16, hipStream_t st) {
   if (nseq < 0 || H < 1 || D < 1 || Dv < 1 || !x || !y || !S || !slots || !positions ||
-      (mode != 0 && mode != 1) || (mode == 0 && !decay) || (mode == 1 && (!N || !M || cap < 0.f)) ||
+      mode < 0 || mode > 2 || (mode == 2 && (R < 1 || !a2t)) || (mode == 0 && !decay) || (mode == 1 && (!N || !M || cap < 0.f)) ||
       rot_dims < 0 || rot_dims > D || (rot_dims & 1) || (rot_dims && !inv_freq) ||
       (gate_act != 0 && gate_act != 1))
     return EIA_BAD_SHAPE;
@@ -242,23 +263,26 @@ EIA_API int eia_linear_scan(const void* x, long ld, int q_off, int k_off, int v_
   if (nseq == 0) return EIA_OK;
   ScanArgs a{x, ld, q_off, k_off, v_off, g_off, i_off, f_off, decay, inv_freq, rot_dims, rot_half,
              qscale, kscale, cap, out_scale, norm_w, S, N, M, slots, cu, positions, seq_lens, y,
-             ldy, eps, H, D, Dv, mode, gate_act};
+             ldy, eps, H, D, Dv, mode, gate_act, lo_off, R, a2t, a2b, inv_tau, norm_h};
   dim3 grid(nseq, H);
-#define LS_LAUNCH(TT, DM, NR)                                                                  \
-  hipLaunchKernelGGL((linear_scan_kernel<TT, DM, NR>), grid, dim3(4 * (DM < 64 ? 64 : DM)), 0, \
+#define LS_LAUNCH(TT, DM, NR, CHN)                                                                  \
+  hipLaunchKernelGGL((linear_scan_kernel<TT, DM, NR, CHN>), grid, dim3(4 * (DM < 64 ? 64 : DM)), 0, \
                      st, a)
-#define LS_SIZES(TT, NR)                      \
-  do {                                        \
-    if (dm <= 32) LS_LAUNCH(TT, 32, NR);      \
-    else if (dm <= 64) LS_LAUNCH(TT, 64, NR); \
-    else if (dm <= 128) LS_LAUNCH(TT, 128, NR); \
-    else LS_LAUNCH(TT, 256, NR);              \
+#define LS_SIZES(TT, NR, CHN)                        \
+  do {                                               \
+    if (dm <= 32) LS_LAUNCH(TT, 32, NR, CHN);        \
+    else if (dm <= 64) LS_LAUNCH(TT, 64, NR, CHN);   \
+    else if (dm <= 128) LS_LAUNCH(TT, 128, NR, CHN); \
+    else LS_LAUNCH(TT, 256, NR, CHN);                \
   } while (0)
-  if (is_bf16) {
-    if (mode == 1) LS_SIZES(bf16_t, true); else LS_SIZES(bf16_t, false);
-  } else {
-    if (mode == 1) LS_SIZES(float, true); else LS_SIZES(float, false);
-  }
+#define LS_MODES(TT)                                 \
+  do {                                               \
+    if (mode == 1) LS_SIZES(TT, true, false);        \
+    else if (mode == 2) LS_SIZES(TT, false, true);   \
+    else LS_SIZES(TT, false, false);                 \
+  } while (0)
+  if (is_bf16) LS_MODES(bf16_t); else LS_MODES(float);
+#undef LS_MODES
 #undef LS_SIZES
 #undef LS_LAUNCH
   EIA_LAUNCH_CHECK();
@@ -273,6 +297,8 @@ EIA_API int eia_linear_scan(const void* x, long ld, int q_off, int k_off, int v_
 //   S_c+1 = exp(A_end) S_c + U_c                            (2) a short scan over a sequence's chunks
 //   o_t   = exp(A_t) S_c^T q_t + sum_(s<=t) exp(A_t - A_s) b_s (q_t . k_s) v_s     (3) per chunk
 //
+// (with a decay per key channel, mode 2, exp(A) is a vector over the channels and acts inside the
+// products: k_s and q_t are scaled channel by channel)
 // (the normaliser n likewise; n_t . q_t is the row sum of the same weights).  Every exponent is
 // <= 0.  The log gates of the gated mode come from a pre-pass that carries the running maximum
 // through the sequence.  All of it fp32 FMA: the 32-bit mode needs it, and the work is small
@@ -286,7 +312,24 @@ struct ChunkArgs {
   const int* seq_first;                     // [nseq + 1]: first chunk of every sequence
   float* wsS; float* wsN; float* wsG;       // [nchunk, H, D, Dv], [nchunk, H, D], [nchunk, H]
   float* la; float* lb; float* nm;          // [rows, H] log a, log b, -m  (mode 1)
-};
+  float* cA;                                // [rows, H * D] running log decays of a chunk (mode 2)
+};                                          // (mode 2: wsG is [nchunk, H, D])
+
+// (A') running log decays per key channel inside every chunk (mode 2), thread = channel.
+template <typename T>
+__global__ void __launch_bounds__(128)
+ls_chan_decay_kernel(ScanArgs a, ChunkArgs c) {
+  const int ch = blockIdx.x, h = blockIdx.y, j = threadIdx.x;
+  const int s = c.chunks[4 * ch], row0 = c.chunks[4 * ch + 1], n = c.chunks[4 * ch + 2];
+  if (a.slots[s] < 0 || j >= a.D) return;
+  const T* X = static_cast<const T*>(a.x);
+  float A = 0.f;
+  for (int t = 0; t < n; ++t) {
+    A += ls_chan_log<T>(a, X + (long)(row0 + t) * a.ld, h, j);
+    c.cA[((long)(row0 + t) * a.H + h) * a.D + j] = A;
+  }
+  c.wsG[((long)ch * a.H + h) * a.D + j] = A;
+}
 
 // (A) log gates of the gated mode: one workgroup per (sequence, head); the transcendentals of 256
 // tokens in parallel, the running maximum serially in one thread.
@@ -383,7 +426,7 @@ EIA_DEV void ls_chunk_decay(const ScanArgs& a, const ChunkArgs& c, int row0, int
 // (1) a chunk's own contribution to the state: U = sum_s w_s k_s v_s^T, u_n = sum_s w_s k_s,
 // w_s = exp(A_end - A_s + log b_s), and the chunk's total log decay.  Thread (r, j): rows
 // [64 r, 64 r + 64) of column j.
-template <typename T>
+template <typename T, bool CH>
 __global__ void __launch_bounds__(256)
 ls_chunk_state_kernel(ScanArgs a, ChunkArgs c) {
   __shared__ __align__(16) float sk[LC][LP], sv[LC][LD];
@@ -399,12 +442,18 @@ ls_chunk_state_kernel(ScanArgs a, ChunkArgs c) {
     sv[t][j] = (t < n && j < Dv) ? ld_f32<T>(X + (long)(row0 + t) * a.ld, a.v_off + (long)h * Dv + j)
                                  : 0.f;
   }
-  ls_chunk_decay(a, c, row0, n, h, sA, sB);
+  if constexpr (!CH) ls_chunk_decay(a, c, row0, n, h, sA, sB);
   __syncthreads();
-  const float Aend = sA[n - 1];
+  const float Aend = CH ? 0.f : sA[n - 1];
   for (int idx = tid; idx < LC * LD; idx += 256) {     // k_s <- w_s k_s
     const int t = idx / LD, j = idx % LD;
-    if (t < n) sk[t][j] *= expf(Aend - sA[t] + sB[t]);
+    if constexpr (CH) {
+      if (t < n && j < D)
+        sk[t][j] *= expf(c.wsG[((long)ch * a.H + h) * D + j] -
+                         c.cA[((long)(row0 + t) * a.H + h) * D + j]);
+    } else {
+      if (t < n) sk[t][j] *= expf(Aend - sA[t] + sB[t]);
+    }
   }
   __syncthreads();
   const int r = tid >> 7, j = tid & 127;
@@ -427,7 +476,7 @@ ls_chunk_state_kernel(ScanArgs a, ChunkArgs c) {
     for (int t = 0; t < n; ++t) un += sk[t][tid];
     c.wsN[((long)ch * a.H + h) * D + tid] = un;
   }
-  if (tid == 0) c.wsG[(long)ch * a.H + h] = Aend;
+  if (!CH && tid == 0) c.wsG[(long)ch * a.H + h] = Aend;
 }
 
 // (2) the scan over a sequence's chunks, element by element: the workspace entry of a chunk turns
@@ -445,12 +494,13 @@ ls_chunk_scan_kernel(ScanArgs a, ChunkArgs c) {
   const long e = (long)blockIdx.z * 256 + threadIdx.x;
   if (e < n_el) {
     float* Sg = a.S + ((long)slot * a.H + h) * n_el;
+    const int ei = (int)(e / a.Dv);                    // state row (key channel)
     float S = fresh ? 0.f : Sg[e];
     for (int ch = c0; ch < c1; ++ch) {
       float* w = c.wsS + ((long)ch * a.H + h) * n_el + e;
       const float U = *w;
       *w = S;
-      S = expf(c.wsG[(long)ch * a.H + h]) * S + U;
+      S = expf(a.mode == 2 ? c.wsG[((long)ch * a.H + h) * a.D + ei] : c.wsG[(long)ch * a.H + h]) * S + U;
     }
     Sg[e] = S;
   }
@@ -469,12 +519,19 @@ ls_chunk_scan_kernel(ScanArgs a, ChunkArgs c) {
 
 // (3) a chunk's outputs from the state before it and its own tokens.  Thread (r, j): tokens
 // r, r + 2, ... of column j.
-template <typename T>
+// CH (a decay per key channel): the pair weights sum q_t k_u exp(A_t - A_u) over the channels.  A
+// chunk is four blocks of eight tokens; pairs inside a block form their exponents one by one,
+// pairs of different blocks factor them through the block edges (E_b: A just before block b),
+//   exp(A_t - A_u) = exp(A_t - E_tb) exp(E_tb - E_(ub+1)) exp(E_(ub+1) - A_u),
+// so every exponent stays <= 0 whatever the decays.
+template <typename T, bool CH>
 __global__ void __launch_bounds__(256)
 ls_chunk_out_kernel(ScanArgs a, ChunkArgs c) {
   __shared__ __align__(16) float sq[LC][LP], sk[LC][LP], sv[LC][LD];
   __shared__ float P[LC][LC + 1];
   __shared__ float sA[LC], sB[LC], snq[LC], red[LC][2];
+  __shared__ __align__(16) float sC[CH ? LC : 1][CH ? LP : 1];   // running log decays per channel
+  __shared__ __align__(16) float sE[CH ? 3 : 1][CH ? LP : 1];    // products over whole blocks
   const int ch = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int s = c.chunks[4 * ch], row0 = c.chunks[4 * ch + 1], n = c.chunks[4 * ch + 2];
   if (a.slots[s] < 0) return;
@@ -487,6 +544,66 @@ ls_chunk_out_kernel(ScanArgs a, ChunkArgs c) {
     sv[t][j] = (t < n && j < Dv) ? ld_f32<T>(X + (long)(row0 + t) * a.ld, a.v_off + (long)h * Dv + j)
                                  : 0.f;
   }
+  if constexpr (CH) {
+    for (int idx = tid; idx < LC * LD; idx += 256) {
+      const int t = idx / LD, j = idx % LD;            // (past the chunk's end: the last token's)
+      sC[t][j] = j < D ? c.cA[((long)(row0 + min(t, n - 1)) * a.H + h) * D + j] : 0.f;
+    }
+    __syncthreads();
+    // pairs inside a block of eight
+    for (int idx = tid; idx < LC * 8; idx += 256) {
+      const int t = idx >> 3, u = (t & ~7) + (idx & 7);
+      float p = 0.f;
+      if (u <= t && t < n) {
+        const f32x4* qa = reinterpret_cast<const f32x4*>(sq[t]);
+        const f32x4* ka = reinterpret_cast<const f32x4*>(sk[u]);
+        const f32x4* At = reinterpret_cast<const f32x4*>(sC[t]);
+        const f32x4* Au = reinterpret_cast<const f32x4*>(sC[u]);
+#pragma unroll 4
+        for (int i = 0; i < (D + 3) / 4; ++i) {
+          const f32x4 x = qa[i] * ka[i], d = At[i] - Au[i];
+          p += x[0] * __expf(d[0]) + x[1] * __expf(d[1]) + x[2] * __expf(d[2]) + x[3] * __expf(d[3]);
+        }
+      }
+      P[t][u] = p;
+    }
+    __syncthreads();
+    // q_t <- q_t exp(A_t - E_tb), k_u <- k_u exp(E_(ub+1) - A_u); block products for the carry
+    for (int idx = tid; idx < LC * LD; idx += 256) {
+      const int t = idx / LD, j = idx % LD, b = t >> 3;
+      const float A = sC[t][j];
+      sq[t][j] *= expf(A - (b ? sC[8 * b - 1][j] : 0.f));
+      sk[t][j] *= expf(sC[8 * b + 7][j] - A);
+      if (t < 3) sE[t][j] = expf(sC[8 * t + 15][j] - sC[8 * t + 7][j]);   // over block t + 1
+    }
+    __syncthreads();
+    // pairs of different blocks: (t, u) with ub < tb, over the blocks between them
+    for (int idx = tid; idx < LC * LC; idx += 256) {
+      const int t = idx / LC, u = idx % LC, tb = t >> 3, ub = u >> 3;
+      if (ub == tb) continue;
+      float p = 0.f;
+      if (ub < tb && t < n) {
+        const f32x4* qa = reinterpret_cast<const f32x4*>(sq[t]);
+        const f32x4* ka = reinterpret_cast<const f32x4*>(sk[u]);
+        const f32x4* e0 = reinterpret_cast<const f32x4*>(sE[ub]);        // block ub + 1
+        const f32x4* e1 = reinterpret_cast<const f32x4*>(sE[ub < 1 ? 1 : ub]);   // block ub + 2
+#pragma unroll 4
+        for (int i = 0; i < (D + 3) / 4; ++i) {
+          f32x4 x = qa[i] * ka[i];
+          if (tb - ub > 1) x *= e0[i];
+          if (tb - ub > 2) x *= e1[i];
+          p += x[0] + x[1] + x[2] + x[3];
+        }
+      }
+      P[t][u] = p;
+    }
+    __syncthreads();
+    // the carry reads q_t exp(A_t)
+    for (int idx = tid; idx < (LC - 8) * LD; idx += 256) {
+      const int t = 8 + idx / LD, j = idx % LD;
+      sq[t][j] *= expf(sC[8 * (t >> 3) - 1][j]);
+    }
+  } else {
   ls_chunk_decay(a, c, row0, n, h, sA, sB);
   __syncthreads();
   // weights of the chunk's own pairs: P[t][u] = (q_t . k_u) exp(A_t - A_u + log b_u), u <= t
@@ -512,6 +629,7 @@ ls_chunk_out_kernel(ScanArgs a, ChunkArgs c) {
     for (int i = 0; i < D; ++i) d += nb[i] * sq[tid][i];
     snq[tid] = d;
   }
+  }
   __syncthreads();
   const int r = tid >> 7, j = tid & 127;
   const float* Sb = c.wsS + ((long)ch * a.H + h) * D * Dv;      // the state before the chunk
@@ -531,13 +649,13 @@ ls_chunk_out_kernel(ScanArgs a, ChunkArgs c) {
     }
   }
   const T* NW = static_cast<const T*>(a.norm_w);
-  const float nw = (NW && j < Dv) ? ld_f32<T>(NW, (long)h * Dv + j) : 1.f;
+  const float nw = (NW && j < Dv) ? ld_f32<T>(NW, (long)h * a.norm_h + j) : 1.f;
   T* Y = static_cast<T*>(a.y);
   const float inv_dv = 1.0f / (float)Dv;
 #pragma unroll
   for (int tt = 0; tt < LC / 2; ++tt) {
     const int t = 2 * tt + r;
-    const float eA = expf(sA[t < n ? t : 0]);
+    const float eA = CH ? 1.f : expf(sA[t < n ? t : 0]);
     float o = (j < Dv && t < n) ? own[tt] + eA * carry[tt] : 0.f;
     if (a.mode == 1 && t < n) {
       float nq = eA * snq[t];
@@ -574,9 +692,12 @@ EIA_API int eia_linear_scan_chunked(const void* x, long ld, int q_off, int k_off
                                     void* y, long ldy, float eps, int nseq, int H, int D, int Dv,
                                     int mode, int gate_act, int is_bf16, const int* chunks,
                                     const int* seq_first, int nchunk, float* wsS, float* wsN,
-                                    float* wsG, float* la, float* lb, float* nm, hipStream_t st) {
+                                    float* wsG, float* la, float* lb, float* nm, int lo_off, int R,
+                                    const float* a2t, const float* a2b, float inv_tau, int norm_h,
+                                    float* cA, hipStream_t st) {
   if (nseq < 0 || nchunk < 0 || H < 1 || D < 1 || Dv < 1 || !x || !y || !S || !slots || !positions ||
-      !chunks || !seq_first || !wsS || !wsG || (mode != 0 && mode != 1) || (mode == 0 && !decay) ||
+      !chunks || !seq_first || !wsS || !wsG || mode < 0 || mode > 2 || (mode == 0 && !decay) ||
+      (mode == 2 && (R < 1 || !a2t || !cA)) ||
       (mode == 1 && (!N || !M || cap < 0.f || !wsN || !la || !lb || !nm)) || rot_dims < 0 ||
       rot_dims > D || (rot_dims & 1) || (rot_dims && !inv_freq) ||
       (gate_act != 0 && gate_act != 1))
@@ -585,19 +706,22 @@ EIA_API int eia_linear_scan_chunked(const void* x, long ld, int q_off, int k_off
   if (nseq == 0 || nchunk == 0) return EIA_OK;
   ScanArgs a{x, ld, q_off, k_off, v_off, g_off, i_off, f_off, decay, inv_freq, rot_dims, rot_half,
              qscale, kscale, cap, out_scale, norm_w, S, N, M, slots, cu, positions, nullptr, y,
-             ldy, eps, H, D, Dv, mode, gate_act};
-  ChunkArgs c{chunks, seq_first, wsS, wsN, wsG, la, lb, nm};
+             ldy, eps, H, D, Dv, mode, gate_act, lo_off, R, a2t, a2b, inv_tau, norm_h};
+  ChunkArgs c{chunks, seq_first, wsS, wsN, wsG, la, lb, nm, cA};
   const dim3 gs(nseq, H), gc(nchunk, H), gz(nseq, H, (D * Dv + 255) / 256);
+#define LS_CHUNKED(TT, CHN)                                                                   \
+  do {                                                                                        \
+    if (mode == 1) hipLaunchKernelGGL((ls_gates_kernel<TT>), gs, dim3(256), 0, st, a, c);     \
+    if (mode == 2) hipLaunchKernelGGL((ls_chan_decay_kernel<TT>), gc, dim3(128), 0, st, a, c); \
+    hipLaunchKernelGGL((ls_chunk_state_kernel<TT, CHN>), gc, dim3(256), 0, st, a, c);         \
+    hipLaunchKernelGGL(ls_chunk_scan_kernel, gz, dim3(256), 0, st, a, c);                     \
+    hipLaunchKernelGGL((ls_chunk_out_kernel<TT, CHN>), gc, dim3(256), 0, st, a, c);           \
+  } while (0)
   if (is_bf16) {
-    if (mode == 1) hipLaunchKernelGGL((ls_gates_kernel<bf16_t>), gs, dim3(256), 0, st, a, c);
-    hipLaunchKernelGGL((ls_chunk_state_kernel<bf16_t>), gc, dim3(256), 0, st, a, c);
-    hipLaunchKernelGGL(ls_chunk_scan_kernel, gz, dim3(256), 0, st, a, c);
-    hipLaunchKernelGGL((ls_chunk_out_kernel<bf16_t>), gc, dim3(256), 0, st, a, c);
+    if (mode == 2) LS_CHUNKED(bf16_t, true); else LS_CHUNKED(bf16_t, false);
   } else {
-    if (mode == 1) hipLaunchKernelGGL((ls_gates_kernel<float>), gs, dim3(256), 0, st, a, c);
-    hipLaunchKernelGGL((ls_chunk_state_kernel<float>), gc, dim3(256), 0, st, a, c);
-    hipLaunchKernelGGL(ls_chunk_scan_kernel, gz, dim3(256), 0, st, a, c);
-    hipLaunchKernelGGL((ls_chunk_out_kernel<float>), gc, dim3(256), 0, st, a, c);
+    if (mode == 2) LS_CHUNKED(float, true); else LS_CHUNKED(float, false);
   }
+#undef LS_CHUNKED
   EIA_LAUNCH_CHECK();
 }

@@ -405,12 +405,30 @@ EIA_API int eia_gnorm(const void* y, long ldy, const float* ypart, int sk, const
 // residual stream.  One launch does, per row,
 //   x += y1 + y2                              (each given or not: sublayer outputs, un-normed)
 //   h  = x / sqrt(mean(x^2) + eps) * w_next   (h != nullptr: the next layer's input)
+//   h  = x                                    (h without w_next: a copy in the activation type)
 // Each y is a stored row (type T, row stride ld) or the fp32 split-K partials [sk, rows, W] of the
-// GEMM that produced it (+ bias), summed here.  A thread re-reads only the columns it wrote, so
+// GEMM that produced it (+ bias), summed here.  A y may have a gate: it then joins as
+// y * sigmoid(g), element by element, g a stored row or W columns of a fused projection's
+// split-K partials (rows gld wide, + bias).  A thread re-reads only the columns it wrote, so
 // the row needs no barrier besides the one inside the sum of squares.
 template <typename T> struct AddRmsSrc {
   const T* y; long ld; const float* part; int sk; const T* bias;
+  const T* g; long ldg; const float* gpart; int gsk; long gld; const T* gbias;
 };
+EIA_DEV float nr_sigmoid(float z) { return 1.0f / (1.0f + __expf(-z)); }
+template <typename T>
+EIA_DEV f32x4 add_rms_gate(const AddRmsSrc<T>& s, long row, int c, long rows) {
+  f32x4 v = {0.f, 0.f, 0.f, 0.f};
+  if (s.g) {
+    v = ld4_f32<T>(s.g + row * s.ldg + c);
+  } else {
+    if (s.gbias) v = ld4_f32<T>(s.gbias + c);
+    const float* p = s.gpart + row * s.gld + c;
+#pragma unroll 4
+    for (int z = 0; z < s.gsk; ++z) v += *reinterpret_cast<const f32x4*>(p + z * rows * s.gld);
+  }
+  return f32x4{nr_sigmoid(v[0]), nr_sigmoid(v[1]), nr_sigmoid(v[2]), nr_sigmoid(v[3])};
+}
 template <typename T>
 EIA_DEV f32x4 add_rms_load(const AddRmsSrc<T>& s, long row, int c, long pstride, int W) {
   f32x4 v = {0.f, 0.f, 0.f, 0.f};
@@ -422,6 +440,7 @@ EIA_DEV f32x4 add_rms_load(const AddRmsSrc<T>& s, long row, int c, long pstride,
 #pragma unroll 4
     for (int z = 0; z < s.sk; ++z) v += *reinterpret_cast<const f32x4*>(p + z * pstride);
   }
+  if (s.g || s.gpart) v *= add_rms_gate<T>(s, row, c, pstride / W);
   return v;
 }
 
@@ -447,13 +466,24 @@ add_rms_kernel(AddRmsSrc<T> s1, AddRmsSrc<T> s2, float* __restrict__ x,
   } else {
     for (int c = threadIdx.x; c < W; c += blockDim.x) {
       float xv = xr[c];
-      if (s1.y) xv += ld_f32<T>(s1.y + row * s1.ld, c);
-      if (s2.y) xv += ld_f32<T>(s2.y + row * s2.ld, c);
+      if (s1.y) xv += ld_f32<T>(s1.y + row * s1.ld, c) *
+                      (s1.g ? nr_sigmoid(ld_f32<T>(s1.g + row * s1.ldg, c)) : 1.f);
+      if (s2.y) xv += ld_f32<T>(s2.y + row * s2.ld, c) *
+                      (s2.g ? nr_sigmoid(ld_f32<T>(s2.g + row * s2.ldg, c)) : 1.f);
       if (any) xr[c] = xv;
       ss += xv * xv;
     }
   }
   if (!h) return;
+  if (!w_next) {                                     // a plain copy
+    if constexpr (VEC) {
+      for (int c = 4 * threadIdx.x; c < W; c += 4 * blockDim.x)
+        st4_f32<T>(h + row * ldh + c, *reinterpret_cast<const f32x4*>(xr + c));
+    } else {
+      for (int c = threadIdx.x; c < W; c += blockDim.x) st_f32<T>(h + row * ldh, c, xr[c]);
+    }
+    return;
+  }
   const float inv = 1.0f / sqrtf(block_sum(ss, scratch) / (float)W + eps);
   if constexpr (VEC) {
     for (int c = 4 * threadIdx.x; c < W; c += 4 * blockDim.x)
@@ -465,24 +495,34 @@ add_rms_kernel(AddRmsSrc<T> s1, AddRmsSrc<T> s2, float* __restrict__ x,
   }
 }
 
-// x fp32 [rows, W] contiguous; y1 / y2, their biases, w_next and h are bf16 when is_bf16 else
-// fp32.  Partials need W % 4 == 0.
+// x fp32 [rows, W] contiguous; y1 / y2, their gates and biases, w_next and h are bf16 when is_bf16
+// else fp32.  Partials need W % 4 == 0.
 EIA_API int eia_add_rms(const void* y1, long ld1, const float* p1, int sk1, const void* b1,
-                        const void* y2, long ld2, const float* p2, int sk2, const void* b2,
-                        float* x, const void* w_next, void* h, long ldh, float eps, int rows, int W,
-                        int is_bf16, hipStream_t st) {
-  if (rows < 0 || W < 1 || !x || (h && !w_next) || (y1 && p1) || (y2 && p2) ||
-      (p1 && (sk1 < 1 || W % 4)) || (p2 && (sk2 < 1 || W % 4)))
+                        const void* g1, long lg1, const float* gp1, int gk1, long gn1,
+                        const void* gb1, const void* y2, long ld2, const float* p2, int sk2,
+                        const void* b2, const void* g2, long lg2, const float* gp2, int gk2,
+                        long gn2, const void* gb2, float* x, const void* w_next, void* h, long ldh,
+                        float eps, int rows, int W, int is_bf16, hipStream_t st) {
+  if (rows < 0 || W < 1 || !x || (y1 && p1) || (y2 && p2) || (w_next && !h) ||
+      (p1 && (sk1 < 1 || W % 4)) || (p2 && (sk2 < 1 || W % 4)) || (g1 && gp1) || (g2 && gp2) ||
+      (gp1 && (gk1 < 1 || gn1 % 4 || reinterpret_cast<uintptr_t>(gp1) % 16)) ||
+      (gp2 && (gk2 < 1 || gn2 % 4 || reinterpret_cast<uintptr_t>(gp2) % 16)))
     return EIA_BAD_SHAPE;
   if (rows == 0) return EIA_OK;
-  const bool vec = W % 4 == 0 && ld1 % 4 == 0 && ld2 % 4 == 0 && ldh % 4 == 0;
-  if (!vec && (p1 || p2)) return EIA_BAD_SHAPE;
+  const int esz = is_bf16 ? 2 : 4;
+  const uintptr_t al = reinterpret_cast<uintptr_t>(g1) | reinterpret_cast<uintptr_t>(g2) |
+                       reinterpret_cast<uintptr_t>(gb1) | reinterpret_cast<uintptr_t>(gb2);
+  const bool vec = W % 4 == 0 && ld1 % 4 == 0 && ld2 % 4 == 0 && ldh % 4 == 0 && lg1 % 4 == 0 &&
+                   lg2 % 4 == 0 && al % (4 * esz) == 0;
+  if (!vec && (p1 || p2 || gp1 || gp2)) return EIA_BAD_SHAPE;
   const int threads = W >= 1024 ? 256 : (W >= 512 ? 128 : 64);
   const long ps = (long)rows * W;
 #define ADD_RMS_LAUNCH(TT, VV)                                                                  \
   do {                                                                                          \
-    AddRmsSrc<TT> a{(const TT*)y1, ld1, p1, sk1, (const TT*)b1};                                \
-    AddRmsSrc<TT> b{(const TT*)y2, ld2, p2, sk2, (const TT*)b2};                                \
+    AddRmsSrc<TT> a{(const TT*)y1, ld1, p1, sk1, (const TT*)b1, (const TT*)g1, lg1, gp1, gk1,   \
+                    gn1, (const TT*)gb1};                                                       \
+    AddRmsSrc<TT> b{(const TT*)y2, ld2, p2, sk2, (const TT*)b2, (const TT*)g2, lg2, gp2, gk2,   \
+                    gn2, (const TT*)gb2};                                                       \
     hipLaunchKernelGGL((add_rms_kernel<TT, VV>), dim3(rows), dim3(threads), 0, st, a, b, x,     \
                        (const TT*)w_next, (TT*)h, ldh, eps, W, ps);                             \
   } while (0)
@@ -492,6 +532,72 @@ EIA_API int eia_add_rms(const void* y1, long ld1, const float* p1, int sk1, cons
     if (vec) ADD_RMS_LAUNCH(float, true); else ADD_RMS_LAUNCH(float, false);
   }
 #undef ADD_RMS_LAUNCH
+  EIA_LAUNCH_CHECK();
+}
+
+// ---------------------------------------------------------------------------------------------
+// The one-group form of the sublayer boundary above gnorm_kernel, a whole workgroup per row:
+//   x += y / sqrt(mean(y^2) + eps) * w_post      (y: a stored row, or split-K partials + bias)
+//   h  = x / sqrt(mean(x^2) + eps) * w_next      (h != nullptr)
+// W, ldy, ldh multiples of 4; a thread re-reads only the columns it wrote.
+template <typename T>
+__global__ void __launch_bounds__(256)
+post_rms_kernel(const T* __restrict__ y, long ldy, const float* __restrict__ ypart, int sk,
+                long pstride, const T* __restrict__ ybias, const T* __restrict__ w_post,
+                float* __restrict__ x, const T* __restrict__ w_next, T* __restrict__ h, long ldh,
+                float eps, int W) {
+  __shared__ float scratch[4];
+  extern __shared__ float ysum[];                    // [W]
+  const long row = blockIdx.x;
+  float* xr = x + row * (long)W;
+  float ss = 0.f;
+  for (int c = 4 * threadIdx.x; c < W; c += 4 * blockDim.x) {
+    f32x4 v = {0.f, 0.f, 0.f, 0.f};
+    if (y) {
+      v = ld4_f32<T>(y + row * ldy + c);
+    } else {
+      if (ybias) v = ld4_f32<T>(ybias + c);
+      const float* p = ypart + row * (long)W + c;
+#pragma unroll 4
+      for (int z = 0; z < sk; ++z) v += *reinterpret_cast<const f32x4*>(p + z * pstride);
+    }
+    *reinterpret_cast<f32x4*>(ysum + c) = v;
+    ss += sumsq4(v);
+  }
+  const float iy = 1.0f / sqrtf(block_sum(ss, scratch) / (float)W + eps);
+  ss = 0.f;
+  for (int c = 4 * threadIdx.x; c < W; c += 4 * blockDim.x) {
+    const f32x4 xv = *reinterpret_cast<const f32x4*>(xr + c) +
+                     *reinterpret_cast<const f32x4*>(ysum + c) * iy * ld4_f32<T>(w_post + c);
+    *reinterpret_cast<f32x4*>(xr + c) = xv;
+    *reinterpret_cast<f32x4*>(ysum + c) = xv;
+    ss += sumsq4(xv);
+  }
+  if (!h) return;
+  const float ix = 1.0f / sqrtf(block_sum(ss, scratch) / (float)W + eps);
+  for (int c = 4 * threadIdx.x; c < W; c += 4 * blockDim.x)
+    st4_f32<T>(h + row * ldh + c,
+               *reinterpret_cast<const f32x4*>(ysum + c) * ix * ld4_f32<T>(w_next + c));
+}
+
+EIA_API int eia_post_rms(const void* y, long ldy, const float* ypart, int sk, const void* ybias,
+                         const void* w_post, float* x, const void* w_next, void* h, long ldh,
+                         float eps, int rows, int W, int is_bf16, hipStream_t st) {
+  if (rows < 0 || W < 1 || W % 4 || ldy % 4 || ldh % 4 || !x || !w_post ||
+      (y == nullptr) == (ypart == nullptr) || (ypart && sk < 1) || (h && !w_next))
+    return EIA_BAD_SHAPE;
+  if ((size_t)W * sizeof(float) > 64 * 1024) return EIA_UNSUPPORTED;
+  if (rows == 0) return EIA_OK;
+  const int threads = W >= 1024 ? 256 : (W >= 512 ? 128 : 64);
+  const long ps = (long)rows * W;
+  if (is_bf16)
+    hipLaunchKernelGGL(post_rms_kernel<bf16_t>, dim3(rows), dim3(threads), sizeof(float) * W, st,
+                       (const bf16_t*)y, ldy, ypart, sk, ps, (const bf16_t*)ybias,
+                       (const bf16_t*)w_post, x, (const bf16_t*)w_next, (bf16_t*)h, ldh, eps, W);
+  else
+    hipLaunchKernelGGL(post_rms_kernel<float>, dim3(rows), dim3(threads), sizeof(float) * W, st,
+                       (const float*)y, ldy, ypart, sk, ps, (const float*)ybias,
+                       (const float*)w_post, x, (const float*)w_next, (float*)h, ldh, eps, W);
   EIA_LAUNCH_CHECK();
 }
 

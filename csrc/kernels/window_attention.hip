@@ -8,11 +8,15 @@
 // value head h / (H / G) of its value columns ([G, Dv]).  For the pair (query position i, key j):
 //
 //   raw_m  = (q_m . k) * mult[m] - slope[m] * (i - j)            (slope == nullptr: no distance term)
+//   raw_m <- cap * tanh(raw_m / cap)                              (cap > 0: soft-capped scores)
 //   s_h    = sum_g talk[h, g] * raw_g                             (talk == nullptr: s = raw)
 //   visible: j <= i and (i - j < window or j < keep)              (window <= 0: every j <= i)
 //   p      = softmax over the visible keys, per map;  a_m = sum_j p_mj v_j
 //   wmode 1: p = sigmoid(s_m + bias[m]) for every visible key, not normalised over the keys
 //            (bias == nullptr: 0; no head mixing, P == 1)
+//   talk_post (wmode 0, P == 1): s = raw; the mixing matrix acts on the softmax weights instead,
+//            p_h <- sum_g talk[h, g] p_g, before the values (scalar form; the matrix-core form of
+//            it is head_mix_attention.hip)
 //   sink (wmode 0, nullable): exp(sink[m]) joins map m's softmax denominator -- a term without a
 //            key or a value, not scaled, counted once.  The running (max, sum) of a row simply
 //            starts at (sink, 1) instead of (-inf, 0); with key partitions, in partition 0.
@@ -257,6 +261,8 @@ struct WinAttnArgs {
   int wmode;                        // 0: softmax; 1: sigmoid(score + bias), un-normalised
   const float* bias;                // [M] or null (wmode 1)
   const float* sink;                // [M] or null (wmode 0)
+  float cap;                        // > 0: scores soft-capped, cap * tanh(s / cap)
+  int talk_post;                    // talk mixes the softmax weights, not the scores (scalar form)
 };
 
 // The visible keys of a 16-query tile as absolute 32-key blocks: the blocks of the kept first
@@ -267,6 +273,10 @@ EIA_DEV WaBlocks wa_blocks(int pos_first, int pos_last, int window, int keep) {
   const int wb0 = lo_min >> 5;
   const int nsink = min((min(keep, lo_min) + 31) >> 5, wb0);
   return WaBlocks{wb0, nsink, nsink + (pos_last >> 5) - wb0 + 1};
+}
+// cap * tanh(s / cap) with icap2 = 2 log2(e) / cap; tanh(x) = 1 - 2 / (exp(2 x) + 1)
+EIA_DEV float wa_softcap(float s, float cap, float icap2) {
+  return cap - 2.f * cap * __builtin_amdgcn_rcpf(exp2f(s * icap2) + 1.f);
 }
 // Key partitions a row really uses: at least two blocks each (a block's dependent chain of
 // loads, products and the exchange is microseconds long, so a lone workgroup should walk few),
@@ -339,6 +349,9 @@ window_attn_kernel(const WinAttnArgs a) {
 #pragma unroll
     for (int i = 0; i < WA_ACC; ++i) acc[i] = 0.f;
 
+    // weights mixed across the heads need every head's final (max, sum): the keys are walked
+    // twice, first for those, then for the weights
+    for (int pass = a.talk_post ? 0 : 1; pass < 2; ++pass)
     for (int k0 = 0; k0 < nkeys; k0 += WA_KT) {
       const int kk = k0 + lane;
       const bool valid = kk < nkeys;
@@ -355,13 +368,24 @@ window_attn_kernel(const WinAttnArgs a) {
         for (int d = 0; d < D; ++d) s += qp[d] * ld_f32<T>(kp, d);
         s *= a.mult[m];
         if (a.slope) s -= a.slope[m] * (float)(pos - j);
+        if (a.cap > 0.f) s = a.cap * tanhf(s / a.cap);
+        if (a.talk_post && pass == 1)                  // the head's own final weight
+          s = valid ? expf(s - mrun[m]) / lrun[m] : 0.f;
         sraw[m * WA_KT + lane] = s;
       }
       __syncthreads();
+      if (a.talk_post && pass == 1) {                  // mix the weights; nothing to rescale
+        for (int m = wave; m < M; m += 4) {
+          float p = 0.f;
+          for (int g = 0; g < M; ++g) p += a.talk[m * M + g] * sraw[g * WA_KT + lane];
+          pw[m * WA_KT + lane] = p;
+          if (lane == 0) alpha[m] = 1.f;
+        }
+      } else {
       // (2) head mixing, mask, online softmax
       for (int m = wave; m < M; m += 4) {
         float s;
-        if (a.talk) {
+        if (a.talk && !a.talk_post) {
           s = 0.f;
           for (int g = 0; g < M; ++g) s += a.talk[m * M + g] * sraw[g * WA_KT + lane];
         } else {
@@ -386,6 +410,8 @@ window_attn_kernel(const WinAttnArgs a) {
           mrun[m] = mn;
         }
       }
+      }
+      if (pass == 0) continue;                         // (uniform)
       __syncthreads();
       // (3) weighted values
       const int nk = min(WA_KT, nkeys - k0);
@@ -408,7 +434,7 @@ window_attn_kernel(const WinAttnArgs a) {
       for (int i = 0; i < WA_ACC; ++i) {
         const int idx = tid + i * 256;
         if (idx < M * Dv) {
-          float v = acc[i] / lrun[idx / Dv] * a.post;
+          float v = (a.talk_post ? acc[i] : acc[i] / lrun[idx / Dv]) * a.post;
           if (gate) v *= 1.0f / (1.0f + expf(-ld_f32<T>(gate + row * a.ldg, idx)));
           st_f32<T>(out + row * a.ldo, idx, v);
         }
@@ -449,8 +475,8 @@ EIA_API int eia_window_attn(const void* q, long ldq, const void* kc, const void*
                             const float* talk, const void* gate, long ldg, void* out, long ldo,
                             int H, int G, int P, int D, int Dv, int bs, int window, int keep,
                             int qb, int epilogue, const float* lam, float eps, float post,
-                            int wmode, const float* bias, const float* sink, int is_bf16,
-                            hipStream_t st) {
+                            int wmode, const float* bias, const float* sink, float cap,
+                            int talk_post, int is_bf16, hipStream_t st) {
   if (n_items < 0 || H < 1 || G < 1 || H % G || (P != 1 && P != 2) || D < 1 || Dv < 1 || bs < 1 ||
       keep < 0 || qb < 1 || !q || !kc || !vc || !bt || !positions || !mult || !out)
     return EIA_BAD_SHAPE;
@@ -458,13 +484,14 @@ EIA_API int eia_window_attn(const void* q, long ldq, const void* kc, const void*
   if ((epilogue == 1) != (P == 2) || (epilogue == 1 && (gate || !lam)))
     return EIA_BAD_SHAPE;
   if ((wmode != 0 && wmode != 1) || (wmode == 1 && (talk || P != 1 || sink))) return EIA_BAD_SHAPE;
+  if (cap < 0.f || (talk_post && (!talk || P != 1 || sink))) return EIA_BAD_SHAPE;
   const int M = H * P;
   const size_t lds = wa_lds_bytes(M, D, Dv);
   if (M * Dv > 256 * WA_ACC || lds > 64 * 1024) return EIA_UNSUPPORTED;
   if (n_items == 0) return EIA_OK;
   WinAttnArgs a{q, ldq, kc, vc, bt, ldbt, positions, cu, work, lens, mult, slope, talk, gate, ldg,
                 out, ldo, H, G, P, D, Dv, bs, window, keep, qb, epilogue, lam, eps, post, 1, 2,
-                nullptr, nullptr, wmode, bias, sink};
+                nullptr, nullptr, wmode, bias, sink, cap, talk_post};
   if (is_bf16)
     hipLaunchKernelGGL((window_attn_kernel<bf16_t>), dim3(n_items), dim3(256), lds, st, a);
   else
@@ -560,6 +587,7 @@ window_attn_mfma_kernel(const WinAttnArgs a) {
     slope[m] = a.slope ? a.slope[hs * P + m] : 0.f;
     sbias[m] = (SIG && a.bias) ? a.bias[hs * P + m] : 0.f;
   }
+  const float cap = a.cap, icap2 = cap > 0.f ? 2.f * LOG2E / cap : 0.f;
   f32x4 acc[MW][NDV];
   float mrun[MW], lrun[MW];
 #pragma unroll
@@ -670,6 +698,13 @@ window_attn_mfma_kernel(const WinAttnArgs a) {
             const int ka = key0 + 8 * g + i;
             s0[i] = s0[i] * mult[m] - slope[m] * (float)(qpos - ka);
             s1[i] = s1[i] * mult[m] - slope[m] * (float)(qpos - ka - 4);
+          }
+          if (cap > 0.f) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+              s0[i] = wa_softcap(s0[i], cap, icap2);
+              s1[i] = wa_softcap(s1[i], cap, icap2);
+            }
           }
           sc[m][0] = s0;
           sc[m][1] = s1;
@@ -928,7 +963,7 @@ EIA_API int eia_window_attn_mfma(const void* q, long ldq, const void* kc, const 
                                  void* out, long ldo, int H, int G, int P, int D, int Dv, int bs,
                                  int window, int keep, int epilogue, const float* lam, float eps,
                                  float post, int wmode, const float* bias, int nparts,
-                                 float* part_acc, float* part_ml, const float* sink,
+                                 float* part_acc, float* part_ml, const float* sink, float cap,
                                  hipStream_t st) {
   if (n_items < 0 || H < 1 || G < 1 || H % G || (P != 1 && P != 2) || bs < 1 || keep < 0 || !q ||
       !kc || !vc || !bt || !positions || !mult || !out)
@@ -937,6 +972,7 @@ EIA_API int eia_window_attn_mfma(const void* q, long ldq, const void* kc, const 
   if ((epilogue == 1) != (P == 2) || (epilogue == 1 && (gate || !lam))) return EIA_BAD_SHAPE;
   if ((wmode != 0 && wmode != 1) || (wmode == 1 && (talk || P != 1 || sink))) return EIA_BAD_SHAPE;
   if (!eia_window_attn_mfma_ok(H, G, P, D, Dv, bs, talk != nullptr)) return EIA_UNSUPPORTED;
+  if (cap < 0.f) return EIA_BAD_SHAPE;
   if (ldq % 8 || ldo % 4) return EIA_BAD_SHAPE;
   // key partitions: decode rows only (a row is its own work item), partials in the workspace
   if (nparts < 1 || nparts > 64 || (nparts > 1 && (cu || !part_acc || !part_ml)))
@@ -944,7 +980,7 @@ EIA_API int eia_window_attn_mfma(const void* q, long ldq, const void* kc, const 
   if (n_items == 0) return EIA_OK;
   WinAttnArgs a{q, ldq, kc, vc, bt, ldbt, positions, cu, work, lens, mult, slope, talk, gate, ldg,
                 out, ldo, H, G, P, D, Dv, bs, window, keep, 16, epilogue, lam, eps, post, nparts,
-                2, part_acc, part_ml, wmode, bias, sink};
+                2, part_acc, part_ml, wmode, bias, sink, cap, 0};
   // raw-score buffers of the head-mixing form: two (one barrier per block) while they fit 48 KiB
   if (talk) a.raw_bufs = (size_t)2 * H * P * 128 * sizeof(f32x4) > 48 * 1024 ? 1 : 2;
   // sigmoid weights: a wave takes two heads of one kv head where the grouping allows it, so the

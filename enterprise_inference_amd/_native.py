@@ -76,10 +76,11 @@ _SIGNATURES = {
                      I, S],
     "eia_moe_route_grouped": [P, L, P, I, I, I, I, I, I, F, P, P, IP, I, I, I, I, P, I, P, P, P, S],
     "eia_linear_scan": [P, L, I, I, I, I, I, I, P, P, I, I, F, F, F, F, P, P, P, P, IP, IP, IP, IP,
-                        P, L, F, I, I, I, I, I, I, I, S],
+                        P, L, F, I, I, I, I, I, I, I, I, P, P, F, I, I, S],
     "eia_moe_finish": [P, L, P, L, P, P, L, P, I, P, P, L, I, I, I, S],
     "eia_linear_scan_chunked": [P, L, I, I, I, I, I, I, P, P, I, I, F, F, F, F, P, P, P, P, IP, IP,
-                                IP, P, L, F, I, I, I, I, I, I, I, IP, IP, I, P, P, P, P, P, P, S],
+                                IP, P, L, F, I, I, I, I, I, I, I, IP, IP, I, P, P, P, P, P, P, I, I,
+                                P, P, F, I, P, S],
     "eia_hyper_step": [P, I, I, P, L, P, I, P, P, P, F, P, P, F, P, L, F, I, I, S],
     "eia_bigram_embed": [IP, P, F, P, I, L, L, IP, IP, IP, I, IP, P, I, I, I, I, I, S],
     "eia_relu2": [P, P, L, I, S],
@@ -89,12 +90,21 @@ _SIGNATURES = {
     "eia_qk_norm_cache": [P, L, P, I, P, I, I, I, I, I, I, I, I, I, P, P, P, L, P, P, P, L, IP, I, F,
                           I, I, S],
     "eia_window_attn": [P, L, P, P, IP, I, IP, IP, IP, IP, I, P, P, P, P, L, P, L, I, I, I, I, I,
-                        I, I, I, I, I, P, F, F, I, P, P, I, S],
+                        I, I, I, I, I, P, F, F, I, P, P, F, I, I, S],
     "eia_window_attn_mfma": [P, L, P, P, IP, I, IP, IP, IP, IP, I, P, P, P, P, L, P, L, I, I, I, I,
-                             I, I, I, I, I, P, F, F, I, P, I, P, P, P, S],
+                             I, I, I, I, I, P, F, F, I, P, I, P, P, P, F, S],
+    "eia_head_mix_attn": [P, L, P, P, IP, I, IP, IP, IP, IP, I, I, P, P, P, L, I, I, I, I, I, I, F,
+                          F, I, P, P, S],
+    "eia_head_mix_attn_ok": [I, I, I, I, I],
+    "eia_qkv_prep": [P, L, P, I, L, P, I, I, I, I, I, I, I, P, P, P, I, P, P, I, I, F, I, F, P, P, I,
+                     IP, IP, IP, IP, IP, I, I, P, L, P, P, I, I, S],
     "eia_qk_rope_cache": [P, L, P, I, P, I, I, I, I, I, I, I, P, P, P, I, I, F, IP, P, L, P, P, IP,
                           I, F, I, I, S],
-    "eia_add_rms": [P, L, P, I, P, P, L, P, I, P, P, P, P, L, F, I, I, I, S],
+    "eia_add_rms": [P, L, P, I, P, P, L, P, I, L, P, P, L, P, I, P, P, L, P, I, L, P, P, P, P, L, F,
+                    I, I, I, S],
+    "eia_post_rms": [P, L, P, I, P, P, P, P, P, L, F, I, I, I, S],
+    "eia_act_mul_embed": [P, L, P, I, L, IP, P, L, I, I, P, I, I, I, I, I, S],
+    "eia_softcap": [P, L, F, S],
     "eia_xielu": [P, L, P, I, L, P, P, L, I, I, I, S],
     "eia_sigmoid_gate": [P, L, L, I, P, L, P, L, I, I, I, S],
     "eia_window_attn_mfma_ok": [I, I, I, I, I, I, I],

@@ -139,20 +139,22 @@ class ModelConfig:
     def from_layer_list(cls, d: Dict[str, Any], name: str = "",
                         tensor_shapes: Optional[Dict[str, Any]] = None) -> "ModelConfig":
         """Designs whose config.json names the architecture in one string and lists the layers
-        one by one (Sekolorn, Vedadra, Gapidra, Daburax): keys ``architecture``, ``vocab``,
-        ``width``, ``norm.eps`` and ``layers`` (kept whole in ``extra["layers"]``); ``norm``,
-        ``embedding`` ({scale, bigram}) and an optional ``loop`` ({start, stop, times}: a run of
-        layers repeated with the same weights) are kept whole too, as are ``residual_mult`` (a
-        factor on every sublayer output) and ``streams`` (residual copies joined by
-        hyper-connections).  Sizes the file leaves to the checkpoint (the rank
-        of a wkv layer's decay branch) come from ``tensor_shapes`` when given."""
+        one by one (Sekolorn, Vedadra, Gapidra, Daburax, Borosun): keys ``architecture``,
+        ``vocab``, ``width``, ``norm.eps`` and ``layers`` (kept whole in ``extra["layers"]``);
+        ``norm``, ``embedding`` ({scale, bigram}) and an optional ``loop`` ({start, stop, times}: a
+        run of layers repeated with the same weights) are kept whole too, as are
+        ``residual_mult`` (a factor on every sublayer output), ``streams`` (residual copies joined
+        by hyper-connections), ``token_side`` ({dim}: a per-layer token embedding) and
+        ``logit_softcap``.  Sizes the file leaves to the checkpoint (the rank of a wkv or gla
+        layer's decay branch) come from ``tensor_shapes`` when given."""
         import copy
         layers = copy.deepcopy(d["layers"])
         for i, L in enumerate(layers):
             m = L.setdefault("mixer", {})
-            if L.get("type") == "wkv" and "decay_rank" not in m:
-                shp = (tensor_shapes or {}).get(f"l{i}.mix.w1")
-                m["decay_rank"] = int(shp[0]) if shp else 64
+            rank = {"wkv": ("w1", 64), "gla": ("a1", 16)}.get(L.get("type"))
+            if rank and "decay_rank" not in m:
+                shp = (tensor_shapes or {}).get(f"l{i}.mix.{rank[0]}")
+                m["decay_rank"] = int(shp[0]) if shp else rank[1]
         heads = [(L["mixer"].get("left") or L["mixer"]).get("heads", 1) for L in layers]
         eps = float((d.get("norm") or {}).get("eps", 1e-6))
         return cls(architecture=d["architecture"], hidden_size=int(d["width"]),
@@ -166,7 +168,9 @@ class ModelConfig:
                                      "embedding": dict(d.get("embedding") or {}),
                                      "loop": dict(d["loop"]) if d.get("loop") else None,
                                      "residual_mult": d.get("residual_mult"),
-                                     "streams": d.get("streams")})
+                                     "streams": d.get("streams"),
+                                     "token_side": dict(d.get("token_side") or {}),
+                                     "logit_softcap": d.get("logit_softcap")})
 
     @classmethod
     def from_hf_dict(cls, d: Dict[str, Any], name: str = "") -> "ModelConfig":

@@ -21,6 +21,7 @@ _REGISTRY: Dict[str, str] = {
     "Vedadra": "vedadra:VedadraForCausalLM",
     "Gapidra": "gapidra:GapidraForCausalLM",
     "Daburax": "daburax:DaburaxForCausalLM",
+    "Borosun": "borosun:BorosunForCausalLM",
     "BertModel": "bert:BertEmbeddingModel",
     "XLMRobertaModel": "bert:BertEmbeddingModel",
     "XLMRobertaForSequenceClassification": "bert:CrossEncoderModel",

@@ -23,12 +23,19 @@ returns the mixer output in the activation dtype.
 * ``SinkAttentionMixer`` -- grouped-query causal softmax attention with projection biases, a
   partial rotation with optional position interpolation and a learned per-head sink in the
   softmax denominator (optionally windowed).
-  All four run on token-major paged K / V rows (``PagedKVRows``, ops/window_attention.py).
+* ``MixAttentionMixer`` -- grouped-query softmax attention whose options are a short causal
+  convolution over time on q, k and v, a weightless RMS norm of the rotated queries and keys, a
+  soft cap on the scores, a sliding window, mixing of the softmax weights across the heads, and
+  value mixing with an earlier layer's values (``ValueCarry``).
+  All five run on token-major paged K / V rows (``PagedKVRows``, ops/window_attention.py).
 * ``RetentionMixer`` -- linear attention with a fixed decay per head: rotated q / k, a matrix
   state per head on per-sequence state slots, head RMS norm, SiLU gate.
 * ``MatrixMemoryMixer`` -- a gated matrix memory: exponential input gate and sigmoid forget gate
   per head with soft-capped pre-activations, stabilised by a running maximum, a normaliser
-  state, head RMS norm with a weight, sigmoid gate.  Both run ops/linear_scan.py.
+  state, head RMS norm with a weight, sigmoid gate.
+* ``GatedLinearMixer`` -- gated linear attention: a matrix state per head whose rows decay per key
+  channel by a data-dependent low-rank branch, head RMS norm with a shared weight, SiLU gate.
+  All three run ops/linear_scan.py.
 * ``ParallelMixer`` -- an attention mixer and a recurrent mixer side by side on the same input:
   one fused input projection, one output projection over the concatenated heads, the two
   outputs added with fixed factors.
@@ -587,7 +594,8 @@ class _ScanMixerBase(nn.Module):
             fused, o["q"][0], o["k"][0], o["v"][0], o["g"][0], self.spec, state, md.seq_slots,
             md.seq_cu, md.num_seqs, md.positions,
             md.decode_seq_lens if md.seq_cu is None else None, norm_w,
-            o["i"][0] if "i" in o else 0, o["f"][0] if "f" in o else 0, out, plan)
+            o["i"][0] if "i" in o else 0, o["f"][0] if "f" in o else 0, out, plan,
+            o["a1"][0] if "a1" in o else 0)
 
     def forward(self, xb: torch.Tensor, md: AttentionMetadata, state):
         # may return gemm.SplitK: the layer's boundary step reduces it
@@ -716,3 +724,135 @@ class ParallelMixer(nn.Module):
         self.right.attend(fused, md, state, out=heads[:, self.lw_pad:self.lw_pad + self.rw])
         # may return gemm.SplitK: the layer's boundary step reduces it
         return gemm.linear(heads, self.o, defer_reduce=True)
+
+
+class ValueCarry:
+    """The values of the first value-mixing layer of a step, [T, kv heads * vdim], handed to the
+    later ones (one object per forward pass; not kept between steps)."""
+
+    __slots__ = ("values",)
+
+    def __init__(self):
+        self.values = None
+
+
+class MixAttentionMixer(_WindowMixerBase):
+    """Grouped-query softmax attention over the part of a caller's fused projection that holds q,
+    k and v (no biases); the caller owns the projection and the output product.  Options:
+
+    * ``taps`` > 1: y_t = sum_j w[c, j] u_(t - taps + 1 + j) on every channel c of q, k and v, zeros
+      before the sequence's start (weights ``q_conv`` / ``k_conv`` / ``v_conv`` [channels, taps]);
+      a state slot keeps each sequence's last taps - 1 projected values
+    * rotation of the first ``rot_dims`` entries of every q / k head (pairs (i, i + rot_dims/2));
+      ``rot_scaling`` as in ops/rotary.py rotary_frequencies
+    * ``qk_norm``: rotated queries and keys are divided by their root mean square per head
+    * score = (q . k) * scale, then cap * tanh(score / cap) with ``softcap``; ``window`` 0 sees
+      every earlier token
+    * ``head_mix``: the softmax weights are mixed, w_h <- sum_g talk[h, g] w_g, before the values
+    * ``v_mix`` "first": the layer's values are the step's ValueCarry; "later": v <- (1 - vmix) v +
+      vmix * carry, and the mixed v is what is cached."""
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, rot_dims: int,
+                 rot_base: float, rot_scaling, eps: float, dtype, device, *, offsets: dict,
+                 taps: int = 1, qk_norm: bool = False, softcap: float = 0.0, window: int = 0,
+                 head_mix: bool = False, v_mix=None):
+        super().__init__()
+        if rot_dims > dim or rot_dims % 2:
+            raise ValueError("rot.dims must be even and at most dim")
+        if not 1 <= taps <= win_ops.PREP_MAX_TAPS:
+            raise ValueError(f"short convolution: 1 .. {win_ops.PREP_MAX_TAPS} taps")
+        if v_mix not in (None, "first", "later"):
+            raise ValueError(f"v_mix {v_mix!r}")
+        self._setup(0, heads, kv_heads, dim, vdim, scale, window, 0, eps, [], False, dtype, device,
+                    norms=False, own_out=False)
+        self.proj = self.proj_bias = None
+        self.offsets = {n: offsets[n] for n in ("q", "k", "v")}
+        inv_freq, amp = rot_ops.rotary_frequencies(rot_dims, rot_base, rot_scaling, device)
+        self.taps, self.v_mix = int(taps), v_mix
+        conv = lambda n: _plain((n, taps), dtype, device) if taps > 1 else None
+        self.q_conv, self.k_conv = conv(heads * dim), conv(kv_heads * dim)
+        self.v_conv = conv(kv_heads * vdim)
+        self.prep = win_ops.PrepSpec(heads, kv_heads, dim, vdim, inv_freq, int(rot_dims), True, amp,
+                                     qk_norm, self.eps, self.taps, self.q_conv, self.k_conv,
+                                     self.v_conv)
+        self.spec.cap = float(softcap)
+        # fp32 copies for the launches, refreshed IN PLACE after a weight load (captured decode
+        # graphs hold their addresses)
+        self.talk = None
+        if head_mix:
+            self.talk = _plain((heads, heads), dtype, device)
+            self.spec.talk = torch.zeros(heads, heads, dtype=torch.float32, device=device)
+            self.spec.talk_post = True
+        self.vmix = self.lam = None
+        if v_mix is not None:                # (the first layer's number is loaded and not used)
+            self.vmix = _param((1,), dtype, device)
+            self.vmix.weight_loader = lambda p, t, sid=None: p.data.copy_(t.reshape(1))
+            self.lam = torch.zeros(1, dtype=torch.float32, device=device)
+
+    @staticmethod
+    def parts(heads, kv_heads, dim, vdim):
+        return [("q", heads * dim), ("k", kv_heads * dim), ("v", kv_heads * vdim)]
+
+    def state_bytes(self, elem: int) -> int:
+        return (self.taps - 1) * self.prep.channels() * elem
+
+    def allocate_state(self, num_slots: int, dtype, device):
+        """[slots, taps - 1, channels] projected values, or None without convolutions."""
+        if self.taps == 1:
+            return None
+        return torch.zeros(max(1, num_slots), self.taps - 1, self.prep.channels(), dtype=dtype,
+                           device=device)
+
+    def refresh(self) -> None:
+        if self.talk is not None:
+            self.spec.talk.copy_(self.talk.float())
+        if self.lam is not None:
+            self.lam.copy_(self.vmix.float())
+
+    def attend(self, fused, md: AttentionMetadata, cache, carry: ValueCarry) -> torch.Tensor:
+        """cache: (PagedKVRows, convolution state or None) -> heads [T, heads * vdim]."""
+        kv, state = cache
+        mode, first = 0, None
+        if self.v_mix == "first":
+            mode = 1
+            first = carry.values = torch.empty(fused.shape[0], self.kv_heads * self.vdim,
+                                               dtype=kv.k.dtype, device=kv.k.device)
+        elif self.v_mix == "later":
+            mode, first = 2, carry.values
+        q = win_ops.qkv_prep_cache(fused, self.offsets["q"][0], self.offsets["k"][0],
+                                   self.offsets["v"][0], self.prep, md, kv.k, kv.v, state,
+                                   self.lam, first, mode)
+        return win_ops.window_attention(q, kv.k, kv.v, md, self.spec, None)
+
+
+class GatedLinearMixer(_ScanMixerBase):
+    """Gated linear attention over a caller's fused projection: q = W_q x * dim^(-1/2), k = W_k x
+    [heads, dim], v = W_v x [heads, vdim]; z = W_a2 (W_a1 x) + bias per head and key channel,
+    alpha = sigmoid(z)^(1/tau);  S_t = diag(alpha_t) S_(t-1) + k_t v_t^T,  o_t = S_t^T q_t; every
+    head's o is RMS-normed and multiplied by ``norm`` [vdim] (shared by the heads); the
+    concatenated heads are multiplied by silu(W_g x)."""
+
+    def __init__(self, heads: int, dim: int, vdim: int, rank: int, tau: float, eps: float, dtype,
+                 device, *, proj: "FusedProjection", prefix: str = ""):
+        super().__init__()
+        self.spec = scan_ops.ScanSpec(heads, dim, vdim, "channel", qscale=float(dim) ** -0.5,
+                                      kscale=1.0, gate_act="silu", eps=float(eps), tau=float(tau),
+                                      norm_shared=True)
+        self._setup(0, self.parts(heads, dim, vdim, rank), (), dtype, device, proj, prefix)
+        self.a2 = _plain((heads * dim, rank), dtype, device)
+        self.a2_bias = _plain((heads * dim,), dtype, device)
+        self.norm = _plain((vdim,), dtype, device)
+        self.spec.a2t = torch.zeros(rank, heads * dim, dtype=torch.float32, device=device)
+        self.spec.a2b = torch.zeros(heads * dim, dtype=torch.float32, device=device)
+
+    @staticmethod
+    def parts(heads, dim, vdim, rank):
+        return [("q", heads * dim), ("k", heads * dim), ("v", heads * vdim), ("g", heads * vdim),
+                ("a1", rank)]
+
+    def refresh(self) -> None:
+        self.spec.a2t.copy_(self.a2.float().t())
+        self.spec.a2b.copy_(self.a2_bias.float())
+
+    def attend(self, fused, md: AttentionMetadata, state, out=None) -> torch.Tensor:
+        return self._scan(fused, md, state, self.norm, out)

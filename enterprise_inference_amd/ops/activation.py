@@ -138,3 +138,48 @@ def sigmoid_gate(a: torch.Tensor, gate: torch.Tensor) -> torch.Tensor:
                                  out.stride(0), T, N, 1 if a.dtype == torch.bfloat16 else 0,
                                  stream(a)), "sigmoid_gate")
     return out
+
+
+def act_mul_embed(u, act: str, ids: torch.Tensor, table: torch.Tensor, col0: int, n: int,
+                  n_pad: int) -> torch.Tensor:
+    """A per-layer token input: act(u[:, :n]) * table[ids, col0:col0 + n] (fp32 inside), zero
+    columns up to ``n_pad`` -> [T, n_pad] in the table's dtype.  ``u`` [T, >= n] is a tensor or a
+    ``gemm.SplitK`` (partial sums of the GEMM that produced it)."""
+    from .gemm import SplitK
+    kind = _KIND[act]
+    split = isinstance(u, SplitK)
+    if split and not (u.part.is_cuda and u.bias is None and u.part.is_contiguous()):
+        u = (u.part.sum(0) + (u.bias.float() if u.bias is not None else 0.0)).to(table.dtype)
+        split = False
+    if not split and not use_hip(u, table):
+        z = u[:, :n].float()
+        a = torch.nn.functional.silu(z) if kind == 0 else \
+            torch.nn.functional.gelu(z, approximate="tanh" if kind == 1 else "none")
+        out = torch.zeros(u.shape[0], n_pad, dtype=table.dtype)
+        out[:, :n] = (a * table[ids[:u.shape[0]].long(), col0:col0 + n].float()).to(table.dtype)
+        return out
+    dt = table.dtype
+    T = u.M if split else u.shape[0]
+    require(dt in (torch.bfloat16, torch.float32) and table.stride(1) == 1 and
+            ids.dtype == torch.int32 and ids.numel() >= T and kind in (0, 1) and
+            0 < n <= n_pad and col0 + n <= table.shape[1], "act_mul_embed: table")
+    require((u.N if split else u.shape[1]) >= n and
+            (split or (u.dtype == dt and u.stride(1) == 1)), "act_mul_embed: rows")
+    out = torch.empty(T, n_pad, dtype=dt, device=table.device)
+    check(lib().eia_act_mul_embed(
+        None if split else ptr(u), 0 if split else u.stride(0), ptr(u.part) if split else None,
+        u.sk if split else 0, u.N if split else 0, ptr(ids), ptr(table), table.stride(0), col0,
+        table.shape[0], ptr(out), T, n, n_pad, kind, 1 if dt == torch.bfloat16 else 0,
+        stream(out)), "act_mul_embed")
+    return out
+
+
+def softcap_(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """x <- cap * tanh(x / cap) in place (fp32, contiguous); cap 0: nothing."""
+    if not cap:
+        return x
+    if not use_hip(x):
+        return x.copy_(cap * torch.tanh(x / cap))
+    require(x.dtype == torch.float32 and x.is_contiguous(), "softcap_: contiguous fp32")
+    check(lib().eia_softcap(ptr(x), x.numel(), float(cap), stream(x)), "softcap")
+    return x

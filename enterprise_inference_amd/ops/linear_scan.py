@@ -1,5 +1,5 @@
-"""Linear-attention recurrences with one decay number per head and token, on per-sequence state
-slots -> csrc/kernels/linear_scan.hip.
+"""Linear-attention recurrences with one decay number per head and token, or one per key channel
+and token, on per-sequence state slots -> csrc/kernels/linear_scan.hip.
 
 Per head a matrix state S [dk, dv] (fp32, slot-resident) that every token scales and adds an
 outer product to; the token's output reads the updated state:
@@ -12,6 +12,9 @@ outer product to; the token's output reads the updated state:
   cap)) (cap 0: i = x_i, f = logsigmoid(x_f)); a running maximum m_t = max(f + m_(t-1), i) (m starts at 0) keeps the exponentials
   bounded: a_t = exp(f + m_(t-1) - m_t), b_t = exp(i - m_t); a normaliser n_t = a_t n_(t-1) +
   b_t k_t divides the output, o_t / (max(|n_t . q_t|, exp(-m_t)) + 1e-6).
+* ``mode="channel"`` (gated linear attention): the row also holds ``rank`` columns of a low-rank
+  branch; z = A2 lo + bias per head and key channel (fp32), a_t = sigmoid(z)^(1/tau) -- a vector
+  that scales the state's rows channel by channel -- and b_t = 1.
 
 q and k may be rotated by the token's position on their first ``rot_dims`` entries and are then
 scaled; every head's output is divided by its root mean square, multiplied by an optional weight,
@@ -47,7 +50,7 @@ class ScanSpec:
     heads: int
     dim: int                        # dk
     vdim: int                       # dv
-    mode: str                       # "decay" | "exp_gates"
+    mode: str                       # "decay" | "exp_gates" | "channel"
     decay: Optional[torch.Tensor] = None        # [H] fp32 ("decay")
     cap: float = 0.0                            # gate soft cap ("exp_gates")
     inv_freq: Optional[torch.Tensor] = None     # [rot_dims / 2] fp32
@@ -58,6 +61,11 @@ class ScanSpec:
     gate_act: str = "silu"          # "silu" | "sigmoid"
     out_scale: float = 1.0
     eps: float = 0.0
+    # "channel": A2 transposed [rank, H*dk] and its bias [H*dk] (fp32, device), tau
+    a2t: Optional[torch.Tensor] = None
+    a2b: Optional[torch.Tensor] = None
+    tau: float = 1.0
+    norm_shared: bool = False       # the weight after the head norm is [dv], shared by the heads
 
 
 class ScanState:
@@ -160,16 +168,19 @@ def linear_scan(fused: torch.Tensor, q_off: int, k_off: int, v_off: int, g_off: 
                 cu: Optional[torch.Tensor], nseq: int, positions: torch.Tensor,
                 seq_lens: Optional[torch.Tensor] = None, norm_w: Optional[torch.Tensor] = None,
                 i_off: int = 0, f_off: int = 0, out: Optional[torch.Tensor] = None,
-                plan: Optional[ChunkPlan] = None) -> torch.Tensor:
+                plan: Optional[ChunkPlan] = None, lo_off: int = 0) -> torch.Tensor:
     """fused [T, *]: rows of one fused projection holding q [H*dk], k [H*dk], v [H*dv], the gate
     [H*dv] (and, with exponential gates, the H input-gate and H forget-gate pre-activations) at
     the given column offsets -> y [T, H*dv] in fused's dtype (``out``: a view to write into).
-    ``norm_w`` [H*dv]: weight after the head RMS norm.  Updates the sequences' slots.
+    ``norm_w`` [H*dv] (or [dv], ``spec.norm_shared``): weight after the head RMS norm.
+    ``lo_off``: first column of the low-rank decay branch ("channel").  Updates the sequences' slots.
     ``plan``: the step's ``chunk_plan`` -- the GPU then runs the chunk-parallel form (heads up to
     128 wide, outside graph capture)."""
     T = fused.shape[0]
     H, D, Dv = spec.heads, spec.dim, spec.vdim
     exp_gates = spec.mode == "exp_gates"
+    channel = spec.mode == "channel"
+    R = spec.a2t.shape[0] if channel else 0
     if out is None:
         out = torch.empty(T, H * Dv, dtype=fused.dtype, device=fused.device)
     require(out.shape == (T, H * Dv) and out.dtype == fused.dtype and out.stride(1) == 1,
@@ -186,6 +197,10 @@ def linear_scan(fused: torch.Tensor, q_off: int, k_off: int, v_off: int, g_off: 
                 (lambda z: z)
             gi = soft(f[:, i_off:i_off + H])
             gf = torch.nn.functional.logsigmoid(soft(f[:, f_off:f_off + H]))
+        if channel:
+            z = f[:, lo_off:lo_off + R] @ spec.a2t.float()
+            z = z + spec.a2b.float() if spec.a2b is not None else z
+            al = torch.exp(torch.nn.functional.logsigmoid(z) / spec.tau).reshape(T, H, D)
         for s, (lo, hi) in enumerate(_seq_bounds(cu, nseq)):
             sl = int(slots[s])
             if hi <= lo or sl < 0:
@@ -206,15 +221,15 @@ def linear_scan(fused: torch.Tensor, q_off: int, k_off: int, v_off: int, g_off: 
                     den = torch.maximum((n * q[t]).sum(-1).abs(), torch.exp(-m)) + 1e-6
                     o = torch.einsum("hi,hij->hj", q[t], S) / den[:, None]
                 else:
-                    S = spec.decay.float()[:, None, None] * S + kv
+                    S = (al[t][:, :, None] if channel else spec.decay.float()[:, None, None]) * S + kv
                     o = torch.einsum("hi,hij->hj", q[t], S)
                 y[t] = o / torch.sqrt((o * o).mean(-1, keepdim=True) + spec.eps)
             state.S[sl] = S
             if exp_gates:
                 state.n[sl], state.m[sl] = n, m
-        y = y.reshape(T, H * Dv)
         if norm_w is not None:
-            y = y * norm_w.float()
+            y = y * (norm_w.float() if spec.norm_shared else norm_w.float().reshape(H, Dv))
+        y = y.reshape(T, H * Dv)
         y = y * (torch.nn.functional.silu(g) if spec.gate_act == "silu" else torch.sigmoid(g))
         out.copy_((y * spec.out_scale).to(out.dtype))
         return out
@@ -223,7 +238,7 @@ def linear_scan(fused: torch.Tensor, q_off: int, k_off: int, v_off: int, g_off: 
     require(fused.stride(1) == 1 and max(q_off + H * D, k_off + H * D, v_off + H * Dv,
                                          g_off + H * Dv) <= fused.shape[1],
             "linear_scan: columns outside the row")
-    require(spec.mode in ("decay", "exp_gates") and spec.gate_act in ("silu", "sigmoid"),
+    require(spec.mode in ("decay", "exp_gates", "channel") and spec.gate_act in ("silu", "sigmoid"),
             "linear_scan: mode")
     require(state.S.dtype == torch.float32 and state.S.is_contiguous() and
             state.S.shape[1:] == (H, D, Dv), "linear_scan: state layout")
@@ -231,6 +246,12 @@ def linear_scan(fused: torch.Tensor, q_off: int, k_off: int, v_off: int, g_off: 
         require(max(i_off, f_off) + H <= fused.shape[1] and state.n is not None and
                 state.m is not None and state.n.is_contiguous() and state.m.is_contiguous() and
                 spec.cap >= 0, "linear_scan: gates")
+    elif channel:
+        require(lo_off + R <= fused.shape[1] and spec.tau > 0 and
+                spec.a2t.shape == (R, H * D) and spec.a2t.is_contiguous() and all(
+                    t is None or (t.dtype == torch.float32 and t.is_cuda)
+                    for t in (spec.a2t, spec.a2b)) and
+                (spec.a2b is None or spec.a2b.numel() == H * D), "linear_scan: channel decays")
     else:
         require(spec.decay is not None and spec.decay.dtype == torch.float32 and
                 spec.decay.is_cuda and spec.decay.numel() == H, "linear_scan: decay per head")
@@ -242,13 +263,18 @@ def linear_scan(fused: torch.Tensor, q_off: int, k_off: int, v_off: int, g_off: 
     require(slots.dtype == torch.int32 and positions.dtype == torch.int32 and
             (cu is None or cu.dtype == torch.int32), "linear_scan: int32 metadata")
     require(norm_w is None or (norm_w.dtype == fused.dtype and norm_w.is_contiguous() and
-                               norm_w.numel() == H * Dv), "linear_scan: norm weight")
+                               norm_w.numel() == (Dv if spec.norm_shared else H * Dv)),
+            "linear_scan: norm weight")
+    mode = {"decay": 0, "exp_gates": 1, "channel": 2}[spec.mode]
+    chan = (lo_off, R, ptr(spec.a2t), ptr(spec.a2b), 1.0 / float(spec.tau),
+            0 if spec.norm_shared else Dv)
     if (plan is not None and plan.n and max(D, Dv) <= CHUNK_MAX_DIM and cu is not None
             and plan.rows == T and (FORCE_CHUNKED or plan.pays(H, max(D, Dv)))
             and not torch.cuda.is_current_stream_capturing()):
         dev = fused.device
         f32 = lambda *shape: torch.empty(*shape, dtype=torch.float32, device=dev)
-        wsS, wsG = f32(plan.n, H, D, Dv), f32(plan.n, H)
+        wsS, wsG = f32(plan.n, H, D, Dv), f32(plan.n, H, D if channel else 1)
+        cA = f32(T, H, D) if channel else None
         wsN = f32(plan.n, H, D) if exp_gates else None
         la, lb, nm = (f32(T, H), f32(T, H), f32(T, H)) if exp_gates else (None, None, None)
         check(lib().eia_linear_scan_chunked(
@@ -257,15 +283,15 @@ def linear_scan(fused: torch.Tensor, q_off: int, k_off: int, v_off: int, g_off: 
             float(spec.qscale), float(spec.kscale), float(spec.cap), float(spec.out_scale),
             ptr(norm_w), ptr(state.S), ptr(state.n), ptr(state.m), ptr(slots), ptr(cu),
             ptr(positions), ptr(out), out.stride(0), float(spec.eps), nseq, H, D, Dv,
-            1 if exp_gates else 0, 0 if spec.gate_act == "silu" else 1, 1 if bf else 0,
+            mode, 0 if spec.gate_act == "silu" else 1, 1 if bf else 0,
             ptr(plan.chunks), ptr(plan.seq_first), plan.n, ptr(wsS), ptr(wsN), ptr(wsG), ptr(la),
-            ptr(lb), ptr(nm), stream(fused)), "linear_scan_chunked")
+            ptr(lb), ptr(nm), *chan, ptr(cA), stream(fused)), "linear_scan_chunked")
         return out
     check(lib().eia_linear_scan(
         ptr(fused), fused.stride(0), q_off, k_off, v_off, g_off, i_off, f_off, ptr(spec.decay),
         ptr(spec.inv_freq), spec.rot_dims, 1 if spec.rot_half else 0, float(spec.qscale),
         float(spec.kscale), float(spec.cap), float(spec.out_scale), ptr(norm_w), ptr(state.S),
         ptr(state.n), ptr(state.m), ptr(slots), ptr(cu), ptr(positions), ptr(seq_lens), ptr(out),
-        out.stride(0), float(spec.eps), nseq, H, D, Dv, 1 if exp_gates else 0,
-        0 if spec.gate_act == "silu" else 1, 1 if bf else 0, stream(fused)), "linear_scan")
+        out.stride(0), float(spec.eps), nseq, H, D, Dv, mode,
+        0 if spec.gate_act == "silu" else 1, *chan, 1 if bf else 0, stream(fused)), "linear_scan")
     return out

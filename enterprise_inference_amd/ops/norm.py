@@ -166,73 +166,104 @@ def group_norm_step(x: torch.Tensor, groups: int, eps: float, y=None,
     if w_next is not None:
         require(w_next.numel() == W, "group_norm_step: weight size")
         h = torch.empty(T, W, dtype=w_next.dtype, device=x.device)
+    if groups == 1 and add is None and (yt is not None or part is not None) and W % 4 == 0 and \
+            (yt is None or yt.stride(0) % 4 == 0) and W <= 16384:
+        # one group: a whole workgroup per row
+        check(lib().eia_post_rms(ptr(yt), yt.stride(0) if yt is not None else 0, ptr(part), sk,
+                                 ptr(ybias), ptr(w_post), ptr(x), ptr(w_next), ptr(h), W,
+                                 float(eps), T, W, 1 if bf else 0, stream(x)), "post_rms")
+        return h
     check(lib().eia_gnorm(ptr(yt), yt.stride(0) if yt is not None else 0, ptr(part), sk,
                           ptr(ybias), ptr(w_post), ptr(x), ptr(add), ptr(w_next), ptr(h), W,
                           float(eps), T, W, groups, 1 if bf else 0, stream(x)), "gnorm")
     return h
 
 
-def residual_rms_step(x: torch.Tensor, eps: float, ys=(), w_next: Optional[torch.Tensor] = None
-                      ) -> Optional[torch.Tensor]:
+def residual_rms_step(x: torch.Tensor, eps: float, ys=(), w_next: Optional[torch.Tensor] = None,
+                      gates=(), copy_dtype: Optional[torch.dtype] = None) -> Optional[torch.Tensor]:
     """Boundary of a layer whose sublayers run side by side on one normed input, around an fp32
     residual stream x [T, W], in one pass over the row:
 
         x += y            for every y in ``ys`` (at most two sublayer outputs, un-normed, in place)
+        x += y * sigmoid(g)     where ``gates`` holds a g for that y
         h  = x / sqrt(mean(x^2) + eps) * w_next      (w_next given: returned in its dtype)
+        h  = x                                       (else copy_dtype given: returned in it)
 
     All arithmetic is fp32.  A y is a tensor in the activation dtype or a ``gemm.SplitK`` (the
-    fp32 partial sums of the GEMM that produced it, plus its bias), reduced here."""
-    from .gemm import SplitK
+    fp32 partial sums of the GEMM that produced it, plus its bias), reduced here; a g is a tensor
+    (W columns, possibly of a wider row) or a ``gemm.SplitKSlice`` of a fused projection."""
+    from .gemm import SplitK, SplitKSlice
     T, W = x.shape
-    ys = [y for y in ys if y is not None]
-    require(len(ys) <= 2, "residual_rms_step: at most two sublayer outputs")
+    gates = list(gates) + [None] * (len(ys) - len(gates))
+    pairs = [(y, g) for y, g in zip(ys, gates) if y is not None]
+    require(len(pairs) <= 2, "residual_rms_step: at most two sublayer outputs")
 
     def dense(y):
         if isinstance(y, SplitK):
             return y.part.sum(0) + (y.bias.float() if y.bias is not None else 0.0)
+        if isinstance(y, SplitKSlice):
+            return y.dense(torch.float32)
         return y.float()
+
+    def joined(y, g):
+        return dense(y) * torch.sigmoid(dense(g)) if g is not None else dense(y)
 
     if use_hip(x) and W % 4:
         # the kernel sums partials in 16-byte units; other widths (no GEMM of the framework
         # produces them) join the stream through the unfused fp32 sum
-        for y in ys:
-            if isinstance(y, SplitK):
-                x += dense(y)
-        ys = [y for y in ys if not isinstance(y, SplitK)]
+        odd = [(y, g) for y, g in pairs if isinstance(y, SplitK) or isinstance(g, SplitKSlice)]
+        for y, g in odd:
+            x += joined(y, g)
+        pairs = [p for p in pairs if not any(p is o for o in odd)]
     if not use_hip(x):
-        for y in ys:
-            x += dense(y)
+        for y, g in pairs:
+            x += joined(y, g)
         if w_next is None:
-            return None
+            return x.to(copy_dtype, copy=True) if copy_dtype is not None else None
         return (x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps) * w_next.float()).to(w_next.dtype)
     require(x.dtype == torch.float32 and x.is_contiguous(), "residual_rms_step: fp32 stream")
-    dt = w_next.dtype if w_next is not None else None
+    dt = w_next.dtype if w_next is not None else copy_dtype
     args = []
-    for y in ys:
+    for y, g in pairs:
         if isinstance(y, SplitK):
             require(y.M == T and y.N == W and y.part.is_contiguous() and
                     y.part.dtype == torch.float32, "residual_rms_step: partials")
             dt = dt or (y.bias.dtype if y.bias is not None else None)
-            args.append((None, 0, y.part, y.sk, y.bias))
+            a = (None, 0, ptr(y.part), y.sk, ptr(y.bias))
+            own = [y.bias]
         else:
             require(y.shape == x.shape and y.stride(-1) == 1, "residual_rms_step: y layout")
             dt = dt or y.dtype
-            require(y.dtype == dt, "residual_rms_step: one activation dtype")
-            args.append((y, y.stride(0), None, 0, None))
-    for a in args:
-        require(a[4] is None or a[4].dtype == dt, "residual_rms_step: bias dtype")
+            a = (ptr(y), y.stride(0), None, 0, None)
+            own = [y]
+        if g is None:
+            a += (None, 0, None, 0, 0, None)
+        elif isinstance(g, SplitKSlice):
+            src = g.src
+            require(src.M == T and g.n == W and g.off % 4 == 0 and src.N % 4 == 0 and
+                    src.part.is_contiguous(), "residual_rms_step: gate partials")
+            b = src.bias[g.off:g.off + W] if src.bias is not None else None
+            a += (None, 0, src.part.data_ptr() + 4 * g.off, src.sk, src.N, ptr(b))
+            own.append(b)
+        else:
+            require(g.shape == x.shape and g.stride(-1) == 1, "residual_rms_step: gate layout")
+            dt = dt or g.dtype
+            a += (ptr(g), g.stride(0), None, 0, 0, None)
+            own.append(g)
+        args.append((a, own))
+    for _, own in args:
+        require(all(t is None or t.dtype == dt for t in own),
+                "residual_rms_step: one activation dtype")
     dt = dt or torch.float32
     require(dt in (torch.bfloat16, torch.float32), "residual_rms_step: bf16 or fp32")
     while len(args) < 2:
-        args.append((None, 0, None, 0, None))
+        args.append(((None, 0, None, 0, None, None, 0, None, 0, 0, None), []))
     h = None
-    if w_next is not None:
-        require(w_next.numel() == W, "residual_rms_step: weight size")
-        h = torch.empty(T, W, dtype=w_next.dtype, device=x.device)
-    (y1, l1, p1, s1, b1), (y2, l2, p2, s2, b2) = args
-    check(lib().eia_add_rms(ptr(y1), l1, ptr(p1), s1, ptr(b1), ptr(y2), l2, ptr(p2), s2, ptr(b2),
-                            ptr(x), ptr(w_next), ptr(h), W, float(eps), T, W,
-                            1 if dt == torch.bfloat16 else 0, stream(x)), "add_rms")
+    if w_next is not None or copy_dtype is not None:
+        require(w_next is None or w_next.numel() == W, "residual_rms_step: weight size")
+        h = torch.empty(T, W, dtype=dt, device=x.device)
+    check(lib().eia_add_rms(*args[0][0], *args[1][0], ptr(x), ptr(w_next), ptr(h), W, float(eps), T,
+                            W, 1 if dt == torch.bfloat16 else 0, stream(x)), "add_rms")
     return h
 
 

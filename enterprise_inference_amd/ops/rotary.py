@@ -74,8 +74,11 @@ def rotary_frequencies(dims: int, base: float, scaling: Optional[dict] = None, d
     multiplied by amp.  f_i = base^(-2i/dims); with ``scaling`` = {factor, original, fast, slow}
     (YaRN) the pairs that turn fewer than ``slow`` times over ``original`` positions are slowed
     by ``factor``, those that turn more than ``fast`` times keep their frequency, the ones
-    between are blended linearly in the pair index, and amp = 0.1 ln(factor) + 1.  A ``scaling``
-    that gives only ``factor`` is linear position interpolation: every f_i is divided by it.
+    between are blended linearly in the pair index, and amp = 0.1 ln(factor) + 1.  With ``scaling``
+    = {factor, original, low, high} (Llama 3.1) the bands are set by wavelength, l = 2 pi / f: below
+    original/high f stays, above original/low it is divided by ``factor``, and between the two
+    blended with s = (original/l - low) / (high - low); amp = 1.  A ``scaling`` that gives only
+    ``factor`` is linear position interpolation: every f_i is divided by it.
     Evaluated in float64 and rounded once."""
     import math
     i = torch.arange(dims // 2, dtype=torch.float64)
@@ -83,6 +86,14 @@ def rotary_frequencies(dims: int, base: float, scaling: Optional[dict] = None, d
     amp = 1.0
     if scaling and "original" not in scaling:
         f = f / float(scaling["factor"])
+    elif scaling and "low" in scaling:
+        factor, orig = float(scaling["factor"]), float(scaling["original"])
+        low, high = float(scaling["low"]), float(scaling["high"])
+        turns = orig * f / (2.0 * math.pi)              # original / wavelength
+        s = (turns - low) / (high - low) if high != low else torch.zeros_like(f)
+        s = torch.where(turns < low, torch.zeros_like(f),
+                        torch.where(turns > high, torch.ones_like(f), s))
+        f = (1.0 - s) * f / factor + s * f
     elif scaling:
         factor, orig = float(scaling["factor"]), float(scaling["original"])
 

@@ -10,6 +10,9 @@ across maps by a matrix (``talk``), masked to ``j <= i and (i-j < window or j < 
 soft-maxed -- or, with ``spec.weights`` 1, every visible key simply weighs
 ``sigmoid(score + bias[m])`` and nothing is normalised over the keys.  With ``spec.sink`` the
 softmax denominator of map m also holds ``exp(sink[m])``, a term without key or value.
+``spec.cap`` > 0 soft-caps the scores, ``cap * tanh(s / cap)``.  With ``spec.talk_post`` the matrix
+``talk`` mixes the softmax WEIGHTS across the heads instead of the scores (each head's mixed
+weights meet its own kv head's values); its matrix-core form is csrc/kernels/head_mix_attention.hip.
 ``spec.epilogue`` 0 multiplies the heads by ``sigmoid(gate)`` and by ``spec.post``; 1 combines
 a head's two maps as ``a1 - lam*a2``, divides by the root mean square over the head and scales.
 
@@ -52,6 +55,8 @@ class WindowSpec:
     weights: int = 0                # 0: softmax over the visible keys; 1: sigmoid(score + bias)
     bias: Optional[torch.Tensor] = None     # [H*P], added to the score inside the sigmoid
     sink: Optional[torch.Tensor] = None     # [H*P], exp(sink) joins the softmax denominator
+    cap: float = 0.0                # > 0: soft cap on the scores
+    talk_post: bool = False         # ``talk`` mixes the softmax weights, not the scores
 
 
 def build_work(q_lens: List[int], qblock: int) -> List[int]:
@@ -71,6 +76,10 @@ def mfma_ok(spec: WindowSpec, dtype: torch.dtype, block_size: int) -> bool:
     the scalar-FMA kernel."""
     if dtype != torch.bfloat16 or not _MFMA_ENV or not torch.cuda.is_available():
         return False
+    if spec.talk_post:
+        return (spec.maps == 1 and spec.keep == 0 and spec.slope is None and
+                bool(lib().eia_head_mix_attn_ok(spec.heads, spec.kv_heads, spec.dim, spec.vdim,
+                                                block_size)))
     return bool(lib().eia_window_attn_mfma_ok(spec.heads, spec.kv_heads, spec.maps, spec.dim,
                                               spec.vdim,
                                               block_size, 1 if spec.talk is not None else 0))
@@ -94,6 +103,18 @@ def decode_partitions(batch: int, spec: WindowSpec, cus: int = 256) -> int:
         limit = max(1, min(16, ((spec.window + 31) // 32 + 1 + (spec.keep + 31) // 32) // 2))
     p = 1
     while p * 2 <= limit and wgs * p * 2 <= 2 * cus:
+        p *= 2
+    return p
+
+
+def head_mix_partitions(batch: int, spec: WindowSpec, cus: int = 256) -> int:
+    """Key partitions of a head-mixing decode launch (a workgroup takes up to 16 heads and four
+    kv heads' values of one row; its four waves split the partition again): a power of two, at
+    most 16, until about two workgroups per CU exist.  Depends on the batch and the layer only."""
+    wgs = max(1, batch) * -(-spec.heads // 16) * -(-spec.kv_heads // 4)
+    blocks = (spec.window + 31) // 32 + 1 if spec.window > 0 else 1 << 20
+    p = 1
+    while p < 16 and wgs * p * 2 <= 2 * cus and p * 8 <= blocks:
         p *= 2
     return p
 
@@ -247,6 +268,154 @@ def qk_rope_cache(fused, q_off: int, k_off: int, v_off: int, mq: int, mk: int, d
     return q
 
 
+PREP_ROWS = 8            # rows per prefill run of qkv_prep_cache (qkv_prep.hip QP_ROWS)
+PREP_MAX_TAPS = 8
+
+
+@dataclasses.dataclass
+class PrepSpec:
+    """Constants of ``qkv_prep_cache`` for one layer."""
+    heads: int
+    kv_heads: int
+    dim: int
+    vdim: int
+    inv_freq: torch.Tensor
+    rot_dims: int = 0
+    rot_half: bool = True
+    rot_amp: float = 1.0
+    norm: bool = False              # every q / k head divided by its root mean square
+    eps: float = 0.0
+    taps: int = 1                   # taps of the short convolutions (1: none)
+    cw_q: Optional[torch.Tensor] = None     # [H*D, taps], [G*D, taps], [G*Dv, taps]
+    cw_k: Optional[torch.Tensor] = None
+    cw_v: Optional[torch.Tensor] = None
+
+    def channels(self) -> int:
+        """Channels of the convolution state: q, k, v columns in this order."""
+        return (self.heads + self.kv_heads) * self.dim + self.kv_heads * self.vdim
+
+
+def _prep_ref(fused, offs, sp: PrepSpec, md, k_cache, v_cache, state, lam, v_first, v_mode):
+    from .latent_attention import _rotate_pairs
+    T = fused.shape[0]
+    H, G, D, Dv, K = sp.heads, sp.kv_heads, sp.dim, sp.vdim, sp.taps
+    f = fused.float()
+    u = torch.cat([f[:, offs[0]:offs[0] + H * D], f[:, offs[1]:offs[1] + G * D],
+                   f[:, offs[2]:offs[2] + G * Dv]], 1)
+    pos = md.positions[:T]
+    if K > 1:
+        w = torch.cat([sp.cw_q, sp.cw_k, sp.cw_v], 0).float()          # [C, taps]
+        cu = md.seq_cu.tolist() if md.seq_cu is not None else list(range(T + 1))
+        y = torch.zeros_like(u)
+        for s in range(len(cu) - 1):
+            lo, hi, sl = cu[s], cu[s + 1], int(md.seq_slots[s])
+            if hi <= lo or sl < 0:
+                continue
+            hist = state[sl].float().clone()                           # [taps - 1, C]
+            p0 = int(pos[lo])
+            if p0 < K - 1:                                             # before the sequence: zeros
+                hist[:K - 1 - p0] = 0
+            ext = torch.cat([hist, u[lo:hi]], 0)
+            for j in range(K):
+                y[lo:hi] += ext[j:j + hi - lo] * w[:, j]
+            state[sl] = ext[-(K - 1):].to(state.dtype)
+        u = y
+    q, k, v = torch.split(u, [H * D, G * D, G * Dv], 1)
+
+    def side(x, m):
+        x = _rotate_pairs(x.reshape(T, m, D), pos[:, None], sp.inv_freq, sp.rot_dims, sp.rot_half,
+                          sp.rot_amp)
+        return (_rms(x, sp.eps) if sp.norm else x).reshape(T, m * D)
+
+    q, k = side(q, H), side(k, G)
+    if v_mode == 1:
+        v_first.copy_(v.to(v_first.dtype))
+    elif v_mode == 2:
+        v = (1.0 - lam.float()) * v + lam.float() * v_first.float()
+    sm = md.slot_mapping[:T].long()
+    ok = sm >= 0
+    k_cache.view(-1, k_cache.shape[-1])[sm[ok]] = k[ok].to(k_cache.dtype)
+    bs = v_cache.shape[2]
+    v_cache[sm[ok] // bs, :, sm[ok] % bs] = v[ok].to(v_cache.dtype)
+    return q.to(k_cache.dtype)
+
+
+def qkv_prep_cache(fused, q_off: int, k_off: int, v_off: int, sp: PrepSpec, md,
+                   k_cache: torch.Tensor, v_cache: torch.Tensor,
+                   state: Optional[torch.Tensor] = None, lam: Optional[torch.Tensor] = None,
+                   v_first: Optional[torch.Tensor] = None, v_mode: int = 0) -> torch.Tensor:
+    """From fused projection rows [T, *] to attention inputs: short causal convolution over time
+    on every channel of q, k and v (``sp.taps`` > 1; ``state`` [slots, taps - 1, channels] holds
+    each sequence's last projected values), rotation of the first ``sp.rot_dims`` entries of every
+    q / k head, an optional weightless RMS norm per head, value mixing, and the cache write.
+    ``v_mode`` 1: the values are also stored in ``v_first`` [T, G*Dv]; 2: v <- (1 - lam) v + lam
+    v_first (``lam`` fp32 [1]).  Returns q [T, H*D].  ``fused`` may be a ``gemm.SplitK``.  A
+    sequence at position 0 starts from zeros whatever its slot held."""
+    from .gemm import SplitK
+    split = isinstance(fused, SplitK)
+    if split and not fused.part.is_cuda:
+        fused = fused.part.sum(0) + (fused.bias.float() if fused.bias is not None else 0.0)
+        split = False
+    H, G, D, Dv = sp.heads, sp.kv_heads, sp.dim, sp.vdim
+    if not split and not use_hip(fused):
+        return _prep_ref(fused, (q_off, k_off, v_off), sp, md, k_cache, v_cache, state, lam,
+                         v_first, v_mode)
+    dt = k_cache.dtype
+    bf = dt == torch.bfloat16
+    require(bf or dt == torch.float32, "qkv_prep_cache: bf16 or fp32")
+    if split:
+        T, width = fused.M, fused.N
+        require(fused.part.dtype == torch.float32 and fused.part.is_contiguous() and
+                (fused.bias is None or fused.bias.dtype == dt), "qkv_prep_cache: partials")
+    else:
+        T, width = fused.shape
+        require(fused.stride(1) == 1 and fused.dtype == dt, "qkv_prep_cache: fused row layout")
+    require(max(q_off + H * D, k_off + G * D, v_off + G * Dv) <= width,
+            "qkv_prep_cache: columns outside the row")
+    require(v_cache.dtype == dt and k_cache.is_contiguous() and v_cache.is_contiguous() and
+            k_cache.shape[-1] == G * D and v_cache.shape[1] == G * Dv and
+            v_cache.shape[2] == k_cache.shape[1], "qkv_prep_cache: cache layout")
+    require(0 <= sp.rot_dims <= D and sp.rot_dims % 2 == 0 and
+            sp.inv_freq.dtype == torch.float32 and sp.inv_freq.numel() >= sp.rot_dims // 2,
+            "qkv_prep_cache: rotation")
+    require(1 <= sp.taps <= PREP_MAX_TAPS, f"qkv_prep_cache: 1 .. {PREP_MAX_TAPS} taps")
+    if sp.taps > 1:
+        for w, rows in ((sp.cw_q, H * D), (sp.cw_k, G * D), (sp.cw_v, G * Dv)):
+            require(w is not None and w.dtype == dt and w.is_contiguous() and
+                    w.shape == (rows, sp.taps), "qkv_prep_cache: convolution weights")
+        require(state is not None and state.dtype == dt and state.is_contiguous() and
+                state.shape[1:] == (sp.taps - 1, sp.channels()) and md.seq_slots is not None and
+                md.seq_slots.dtype == torch.int32, "qkv_prep_cache: convolution state")
+    require(v_mode == 0 or (v_first is not None and v_first.dtype == dt and
+                            v_first.is_contiguous() and v_first.shape == (T, G * Dv)),
+            "qkv_prep_cache: first values")
+    require(v_mode != 2 or (lam is not None and lam.dtype == torch.float32), "qkv_prep_cache: lam")
+    require(md.slot_mapping.dtype == torch.int32 and md.slot_mapping.numel() >= T and
+            md.positions.dtype == torch.int32 and md.positions.numel() >= T,
+            "qkv_prep_cache: int32 slots and positions")
+    q = torch.empty(T, H * D, dtype=dt, device=k_cache.device)
+    nd = md.num_decode
+
+    def launch(base, n_items, cu, work):
+        sl = md.seq_slots[base:] if (md.seq_slots is not None and sp.taps > 1) else None
+        check(lib().eia_qkv_prep(
+            None if split else ptr(fused), width if split else fused.stride(0),
+            ptr(fused.part) if split else None, fused.sk if split else 0, T * width if split else 0,
+            ptr(fused.bias) if split else None, q_off, k_off, v_off, H, G, D, Dv, ptr(sp.cw_q),
+            ptr(sp.cw_k), ptr(sp.cw_v), sp.taps, ptr(state), ptr(sp.inv_freq), sp.rot_dims,
+            1 if sp.rot_half else 0, float(sp.rot_amp), 1 if sp.norm else 0, float(sp.eps),
+            ptr(lam), ptr(v_first), v_mode, ptr(md.positions), ptr(md.slot_mapping), ptr(sl),
+            ptr(cu), ptr(work), base, n_items, ptr(q), q.stride(0), ptr(k_cache), ptr(v_cache),
+            k_cache.shape[1], 1 if bf else 0, stream(q)), "qkv_prep")
+
+    if nd:
+        launch(0, nd, None, None)
+    if md.num_prefill_tokens:
+        work, n_work = md.prefill_work_for(PREP_ROWS, build_work)
+        launch(nd, n_work, md.prefill_cu_q, work)
+    return q
+
+
 def _ref_rows(q, k_cache, v_cache, block_table, positions, gate, spec: WindowSpec, seq_of_row):
     """Plain per-row attention over the paged rows (CPU path)."""
     H, G, P, D, Dv = spec.heads, spec.kv_heads, spec.maps, spec.dim, spec.vdim
@@ -265,7 +434,9 @@ def _ref_rows(q, k_cache, v_cache, block_table, positions, gate, spec: WindowSpe
         sc = torch.einsum("md,nmd->mn", q[row].float().view(H * P, D), keys) * spec.mult[:, None]
         if spec.slope is not None:
             sc = sc - spec.slope[:, None] * (i - js).float()[None, :]
-        if spec.talk is not None:
+        if spec.cap > 0:
+            sc = spec.cap * torch.tanh(sc / spec.cap)
+        if spec.talk is not None and not spec.talk_post:
             sc = spec.talk @ sc
         if spec.weights == 1:
             w = torch.sigmoid(sc + (spec.bias[:, None] if spec.bias is not None else 0.0))
@@ -273,6 +444,8 @@ def _ref_rows(q, k_cache, v_cache, block_table, positions, gate, spec: WindowSpe
             w = torch.softmax(torch.cat([sc, spec.sink[:, None]], -1), -1)[:, :-1]
         else:
             w = torch.softmax(sc, -1)
+        if spec.talk_post:
+            w = spec.talk @ w
         w = w.view(H, P, len(js))
         a = torch.einsum("hpn,nhd->hpd", w, vals)
         if spec.epilogue == 0:
@@ -324,6 +497,9 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
     require(spec.weights in (0, 1) and (spec.weights == 0 or (spec.talk is None and P == 1)),
             "window_attention: sigmoid weights come without head mixing or map pairs")
     require(spec.sink is None or spec.weights == 0, "window_attention: a sink needs softmax weights")
+    require(not spec.talk_post or (spec.talk is not None and P == 1 and spec.weights == 0 and
+                                   spec.sink is None and gate is None and spec.epilogue == 0),
+            "window_attention: mixed weights come with a plain softmax, one map per head, no gate")
     for t in (spec.mult, spec.slope, spec.talk, spec.lam, spec.bias, spec.sink):
         require(t is None or (t.dtype == torch.float32 and t.is_cuda and t.is_contiguous()),
                 "window_attention: fp32 device constants")
@@ -337,6 +513,19 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         require(bt.dtype == torch.int32 and bt.stride(1) == 1, "block tables int32")
         qa, o = q[lo:], out[lo:]
         g = None if gate is None else gate[lo:]
+        if mfma and spec.talk_post:
+            rows = n_items if cu is None else T - lo
+            NP = head_mix_partitions(n_items, spec) if cu is None else 1
+            acc = torch.empty(rows * NP * H * spec.kv_heads * Dv, dtype=torch.float32,
+                              device=q.device)
+            ml = torch.empty(rows * NP * H * 2, dtype=torch.float32, device=q.device)
+            check(lib().eia_head_mix_attn(
+                ptr(qa), qa.stride(0), ptr(k_cache), ptr(v_cache), ptr(bt), bt.stride(0),
+                ptr(md.positions[lo:]), ptr(cu), ptr(work), ptr(lens), n_items, rows,
+                ptr(spec.mult), ptr(spec.talk), ptr(o), o.stride(0), H, spec.kv_heads, D, Dv, bs,
+                spec.window, float(spec.cap), float(spec.post), NP, ptr(acc), ptr(ml), stream(q)),
+                "head_mix_attn")
+            return
         if mfma:
             NP = decode_partitions(n_items, spec) if cu is None else 1
             pa = pm = None
@@ -349,7 +538,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                 ptr(spec.slope), ptr(spec.talk), ptr(g), g.stride(0) if g is not None else 0,
                 ptr(o), o.stride(0), H, spec.kv_heads, P, D, Dv, bs, spec.window, spec.keep,
                 spec.epilogue, ptr(spec.lam), float(spec.eps), float(spec.post), spec.weights,
-                ptr(spec.bias), NP, ptr(pa), ptr(pm), ptr(spec.sink), stream(q)), "window_attn_mfma")
+                ptr(spec.bias), NP, ptr(pa), ptr(pm), ptr(spec.sink), float(spec.cap),
+                stream(q)), "window_attn_mfma")
             return
         check(lib().eia_window_attn(
             ptr(qa), qa.stride(0), ptr(k_cache), ptr(v_cache), ptr(bt), bt.stride(0),
@@ -357,7 +547,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
             ptr(spec.slope), ptr(spec.talk), ptr(g), g.stride(0) if g is not None else 0, ptr(o),
             o.stride(0), H, spec.kv_heads, P, D, Dv, bs, spec.window, spec.keep, qb,
             spec.epilogue, ptr(spec.lam), float(spec.eps), float(spec.post), spec.weights,
-            ptr(spec.bias), ptr(spec.sink), 1 if bf else 0, stream(q)), "window_attn")
+            ptr(spec.bias), ptr(spec.sink), float(spec.cap), 1 if spec.talk_post else 0,
+            1 if bf else 0, stream(q)), "window_attn")
 
     if nd:
         launch(0, nd, md.decode_block_tables, md.decode_seq_lens, None, None, 1)
