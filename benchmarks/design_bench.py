@@ -18,6 +18,11 @@ and parallel layers of sink attention beside a gated matrix memory; a group-limi
 gated experts with identity experts and a gated shared expert) beside Sekolorn, the closest
 existing design (recurrent and attention layers on state slots and paged rows, a group-routed
 mixture of experts with a shared expert), at equal width, depth, heads, experts and expert ff.
+``--design borosun`` runs the Borosun design (parallel sublayers with gated residuals and a
+per-layer token input; head-mixed full attention behind short convolutions, soft-capped window
+attention, gated linear attention) beside Gapidra, the closest existing design (parallel
+sublayers on one norm, window attention, dense feed-forward), at equal width, depth, heads, head
+size, window and ff.
 Prefill: ``--design-prompts`` prompts of ``--design-prompt-len`` tokens, one sampled token each.
 Decode: ``--design-users`` sequences of 128 prompt tokens generating ``--design-gen`` tokens; the
 decode rate is the extra tokens over the extra time against the same run with one token.
@@ -168,6 +173,32 @@ def daburax_config(z: dict) -> dict:
             "layers": [ret, ret, par] * (z["layers"] // 3)}
 
 
+BSIZES = {
+    # Gapidra's sizes, the side width, the gla heads (keys half as wide as values)
+    "bs": dict(GSIZES["gs"], layers=6, side=128),
+    "bm": dict(GSIZES["gm"], layers=6, side=256),
+}
+
+
+def borosun_config(z: dict) -> dict:
+    H, G, D = z["heads"], z["kv_heads"], z["dim"]
+    mlp = {"kind": "dense", "ff": z["ff"]}
+    att = {"type": "attention", "mlp": mlp,
+           "mixer": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5, "conv": 3,
+                     "v_mix": True,
+                     "rot": {"base": 5e5, "dims": D, "scaling": {"factor": 8.0, "low": 1.0,
+                                                                 "high": 4.0, "original": 8192}}}}
+    att2 = {"type": "attention_2", "mlp": mlp,
+            "mixer": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5,
+                      "softcap": 50.0, "v_mix": True, "mask": {"size": z["window"]},
+                      "rot": {"base": 1e4, "dims": D // 2}}}
+    gla = {"type": "gla", "mlp": mlp,
+           "mixer": {"heads": H, "dim": D // 2, "vdim": D, "tau": 8.0, "decay_rank": 16}}
+    return {"architecture": "Borosun", "vocab": z["vocab"], "width": z["width"],
+            "norm": {"eps": 1e-5}, "token_side": {"dim": z["side"]}, "logit_softcap": 30.0,
+            "layers": [att, att2, gla] * (z["layers"] // 3)}
+
+
 def sekolorn_like(z: dict) -> dict:
     """Sekolorn at a Daburax size: same width, depth, heads, experts, top-k and expert ff."""
     return sekolorn_config(dict(width=z["width"], layers=z["layers"], heads=z["heads"], dim=64,
@@ -227,7 +258,8 @@ def run(a) -> int:
     rows = []
     design = getattr(a, "design", "sekolorn")
     vedadra = design == "vedadra"
-    default = {"vedadra": "vs,vm", "gapidra": "gs,gm", "daburax": "ds,dm"}.get(design, "s,s6")
+    default = {"vedadra": "vs,vm", "gapidra": "gs,gm", "daburax": "ds,dm",
+               "borosun": "bs,bm"}.get(design, "s,s6")
     for name in (a.design_sizes or default).split(","):
         if name in GATED:
             raise SystemExit(f"design size {name!r} is switched off (see GATED in "
@@ -239,6 +271,9 @@ def run(a) -> int:
             other = ("Sekolorn", sekolorn_like(z)) if name == "ds" else \
                 ("Mixtral-style", mixtral_config(z))
             pair = (("Daburax", daburax_config(z)), other)
+        elif design == "borosun":
+            z = BSIZES[name]
+            pair = (("Borosun", borosun_config(z)), ("Gapidra", gapidra_config(z)))
         elif design == "gapidra":
             z = dict(GSIZES[name], layers=6)
             pair = (("Gapidra", gapidra_config(z)), ("Mistral-style", mistral_config(z)))
@@ -291,6 +326,8 @@ def kernel_rates(a) -> int:
         return gapidra_kernel_rates(a)
     if getattr(a, "design", "sekolorn") == "daburax":
         return daburax_kernel_rates(a)
+    if getattr(a, "design", "sekolorn") == "borosun":
+        return borosun_kernel_rates(a)
     from enterprise_inference_amd.ops import attention as A
     from enterprise_inference_amd.ops import latent_attention as LA
     from enterprise_inference_amd.ops import wkv as WK
@@ -764,5 +801,168 @@ def daburax_kernel_rates(a) -> int:
                      "ms": t * 1e3, "GBps": Tn * W * 2 / t / 1e9})
     for r_ in rows:
         print(json.dumps(r_), flush=True)
+    print(json.dumps({"metric": "design_kernel_rates", "rows": rows}), flush=True)
+    return 0
+
+
+def borosun_kernel_rates(a) -> int:
+    """Achieved rates of the Borosun kernels beside their like kernels at equal heads and lengths.
+    Attention in useful TFLOP/s (2 (Dqk + Dv) per visible query-key pair and head; the extra value
+    products of the head mixing are reported as their own rate) and, at decode, cache bytes of the
+    visible keys per second: head-mixed attention beside the same window-attention family with the
+    scores mixed (Vedadra's mixer) and with a plain softmax, soft-capped window attention beside
+    sigmoid window attention (Gapidra's mixer).  The per-channel linear scan beside the fixed-decay
+    one and the wkv scan (tokens/s, state bytes/s).  The prep kernel, the gated boundary and the
+    side output beside their like kernels in bytes moved per second.  One JSON line per kernel."""
+    import torch
+
+    from enterprise_inference_amd.ops import activation as AC
+    from enterprise_inference_amd.ops import attention as A
+    from enterprise_inference_amd.ops import linear_scan as LS
+    from enterprise_inference_amd.ops import norm as N
+    from enterprise_inference_amd.ops import window_attention as WA
+    from enterprise_inference_amd.ops import wkv as WK
+    from enterprise_inference_amd.ops.rotary import rotary_frequencies
+
+    dev, bf = "cuda", torch.bfloat16
+    rows = []
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=dev)
+    bs, T, win, D = 128, 4096, 1024, 128
+    full = T * (T + 1) // 2
+    wpairs = T * win - win * (win - 1) // 2
+    B, L = 64, 4096
+    nb, nbd = T // bs, B * L // bs
+    pos = torch.arange(T, dtype=torch.int32, device=dev)
+    bt = torch.arange(nb, dtype=torch.int32, device=dev)[None]
+    wl = A.build_prefill_work([T], WA.MFMA_QB)
+    md = A.AttentionMetadata(
+        num_decode=0, num_prefill_tokens=T, slot_mapping=pos, positions=pos,
+        prefill_block_tables=bt, prefill_seq_lens=i32([T]), prefill_cu_q=i32([0, T]),
+        prefill_q_lens=[T], prefill_work=i32(wl), prefill_n_work=len(wl) // 2,
+        prefill_qblock=WA.MFMA_QB, num_seqs=1, seq_slots=i32([0]), seq_cu=i32([0, T]))
+    posd = torch.full((B,), L - 1, dtype=torch.int32, device=dev)
+    btd = torch.arange(nbd, dtype=torch.int32, device=dev).view(B, L // bs)
+    mdd = A.AttentionMetadata(num_decode=B, num_prefill_tokens=0, slot_mapping=btd[:, -1] * bs + bs - 1,
+                              positions=posd, decode_block_tables=btd, decode_seq_lens=i32([L] * B),
+                              num_seqs=B, seq_slots=torch.arange(B, dtype=torch.int32, device=dev))
+    for H, G in ((8, 2), (16, 4)):
+        mult = torch.full((H,), D ** -0.5, device=dev)
+        talk = torch.eye(H, device=dev) + 0.1 * torch.randn(H, H, device=dev)
+        mk = lambda **k: WA.WindowSpec(H, G, 1, D, D, k.pop("window", 0), 0, mult=mult, **k)
+        kinds = [("head-mixed weights, causal", mk(talk=talk, talk_post=True), full, L),
+                 ("head-mixed scores, causal", mk(talk=talk), full, L),
+                 ("plain softmax, causal", mk(), full, L),
+                 ("soft cap, window", mk(cap=50.0, window=win), wpairs, win),
+                 ("sigmoid weights, window", mk(weights=1, bias=torch.zeros(H, device=dev),
+                                                window=win), wpairs, win)]
+        kc = torch.randn(nb, bs, G * D, device=dev).to(bf)
+        vc = torch.randn(nb, G * D, bs, device=dev).to(bf)
+        q = torch.randn(T, H * D, device=dev).to(bf)
+        kcd = torch.randn(nbd, bs, G * D, device=dev).to(bf)
+        vcd = torch.randn(nbd, G * D, bs, device=dev).to(bf)
+        qd = q[:B].contiguous()
+        for label, spec, pairs, keys in kinds:
+            t = _time(lambda: WA.window_attention(q, kc, vc, md, spec, None))
+            r = {"kernel": f"attention prefill ({label})", "heads": H, "kv_heads": G, "dim": D,
+                 "tokens": T, "ms": t * 1e3, "mfma": WA.mfma_ok(spec, bf, bs),
+                 "tflops": 2.0 * 2 * D * H * pairs / t / 1e12}
+            if spec.talk_post:      # all products formed: every head against every kv head's values
+                r["tflops_formed"] = 2.0 * D * (1 + G) * H * pairs / t / 1e12
+            rows.append(r)
+            t = _time(lambda: WA.window_attention(qd, kcd, vcd, mdd, spec, None))
+            rows.append({"kernel": f"attention decode ({label})", "heads": H, "kv_heads": G,
+                         "batch": B, "context": L, "ms": t * 1e3,
+                         "cache_GBps": B * keys * G * 2 * D * 2 / t / 1e9})
+        # ---- projection rows to attention inputs
+        inv, _ = rotary_frequencies(D, 1e4, None, dev)
+        width = (H + 2 * G) * D + 2 * H * D
+        fused = torch.randn(T, width, device=dev).to(bf)
+        cw = lambda n: torch.randn(n, 4, device=dev).to(bf)
+        for taps in (1, 4):
+            sp = WA.PrepSpec(H, G, D, D, inv, D, True, 1.0, False, 1e-6, taps, cw(H * D)[:, :taps]
+                             .contiguous(), cw(G * D)[:, :taps].contiguous(),
+                             cw(G * D)[:, :taps].contiguous())
+            st = torch.zeros(B, max(1, taps - 1), sp.channels(), device=dev).to(bf)
+            t = _time(lambda: WA.qkv_prep_cache(fused, 0, H * D, (H + G) * D, sp, md, kc, vc,
+                                                st if taps > 1 else None))
+            rows.append({"kernel": f"qkv_prep ({taps} taps)", "heads": H, "kv_heads": G, "rows": T,
+                         "ms": t * 1e3, "GBps": T * (H + 2 * G) * D * 4 / t / 1e9})
+        t = _time(lambda: WA.qk_rope_cache(fused, 0, H * D, (H + G) * D, H, G, D, G * D, None, None,
+                                           inv, D, True, 1.0, pos, kc, vc, pos, 1e-6))
+        rows.append({"kernel": "qk_rope_cache", "heads": H, "kv_heads": G, "rows": T, "ms": t * 1e3,
+                     "GBps": T * (H + 2 * G) * D * 4 / t / 1e9})
+        del kcd, vcd
+    # ---- scans
+    for Hh, Dk, Dv in ((32, 64, 64), (16, 64, 128), (16, 128, 128)):
+        for nseq, per in ((1, 4096), (4, 2048), (64, 1)):
+            Tn = nseq * per
+            slots = torch.arange(nseq, dtype=torch.int32, device=dev)
+            cu = torch.arange(0, Tn + 1, per, dtype=torch.int32, device=dev)
+            ps = (torch.arange(Tn, dtype=torch.int32, device=dev) % per) + (5 if per == 1 else 0)
+            R = 16
+            x = (torch.randn(Tn, 2 * Hh * Dk + 2 * Hh * Dv + R, device=dev) * 0.3).to(bf)
+            nw = torch.ones(Dv, device=dev).to(bf)
+            for mode in ("channel", "decay"):
+                spec = LS.ScanSpec(Hh, Dk, Dv, mode, decay=torch.full((Hh,), 0.97, device=dev),
+                                   qscale=Dk ** -0.5, gate_act="silu", eps=1e-5, tau=16.0,
+                                   a2t=torch.randn(R, Hh * Dk, device=dev) * 0.2,
+                                   a2b=torch.ones(Hh * Dk, device=dev), norm_shared=True)
+                st = LS.ScanState.allocate(nseq, spec, dev)
+                forms = [("token by token", None)]
+                if per > 1:
+                    forms.append(("chunk-parallel", LS.chunk_plan([per] * nseq, dev)))
+                for form, plan in forms:
+                    LS.FORCE_CHUNKED = plan is not None
+                    c = (0, Hh * Dk, 2 * Hh * Dk, 2 * Hh * Dk + Hh * Dv)
+                    t = _time(lambda: LS.linear_scan(x, *c, spec, st, slots, cu if per > 1 else None,
+                                                     nseq, ps, None, nw, plan=plan,
+                                                     lo_off=2 * Hh * (Dk + Dv)))
+                    rows.append({"kernel": f"linear_scan ({mode}, {form})", "heads": Hh,
+                                 "dim": [Dk, Dv], "seqs": nseq, "tokens_per_seq": per,
+                                 "ms": t * 1e3, "tokens_per_s": Tn / t,
+                                 "state_GBps": nseq * Hh * Dk * Dv * 4 * 2 / t / 1e9})
+                LS.FORCE_CHUNKED = False
+            if (Dk, Dv) == (64, 64):
+                HD, W = Hh * 64, 2048
+                r_, k, v, g = (torch.randn(Tn, HD, device=dev).to(bf) * 0.3 for _ in range(4))
+                dec = torch.randn(Tn, HD, device=dev) * 0.3
+                w0 = torch.full((HD,), -1.0, device=dev).to(bf)
+                u = (torch.randn(HD, device=dev) * 0.3).to(bf)
+                nw = torch.ones(HD, device=dev).to(bf)
+                S = torch.zeros(nseq, Hh, 64, 64, device=dev)
+                prev = torch.zeros(nseq, W, device=dev)
+                xx = torch.randn(Tn, W, device=dev)
+                t = _time(lambda: WK.wkv_scan(r_, k, v, g, dec, w0, u, nw, S, prev, xx, slots, cu,
+                                              nseq, ps, None, 1e-5, Hh))
+                rows.append({"kernel": "wkv_scan", "heads": Hh, "dim": 64, "seqs": nseq,
+                             "tokens_per_seq": per, "ms": t * 1e3, "tokens_per_s": Tn / t,
+                             "state_GBps": nseq * Hh * 64 * 64 * 4 * 2 / t / 1e9})
+    # ---- layer boundary
+    for W, side in ((1024, 128), (2048, 256)):
+        Tn = 8192
+        x = torch.randn(Tn, W, device=dev)
+        y1, y2 = torch.randn(Tn, W, device=dev).to(bf), torch.randn(Tn, W, device=dev).to(bf)
+        gt = torch.randn(Tn, 2 * W, device=dev).to(bf)
+        w1 = torch.ones(W, device=dev).to(bf)
+        ids = torch.randint(0, 32000, (Tn,), device=dev).to(torch.int32)
+        tab = torch.randn(32000, 6 * side, device=dev).to(bf)
+        u = torch.randn(Tn, side, device=dev).to(bf)
+        cases = [("gated residual sum", W * (8 + 4 * 2 + 2),
+                  lambda: N.residual_rms_step(x, 1e-6, (y1, y2), None, (gt[:, :W], gt[:, W:]),
+                                              copy_dtype=bf)),
+                 ("residual sum + norm (no gates)", W * (8 + 2 * 2 + 2),
+                  lambda: N.residual_rms_step(x, 1e-6, (y1, y2), w1)),
+                 ("side output norm + next norm", W * (8 + 2 + 2),
+                  lambda: N.group_norm_step(x, 1, 1e-6, y1, w1, None, w1)),
+                 ("output norm + next norm, 4 groups", W * (8 + 2 + 2),
+                  lambda: N.group_norm_step(x, 4, 1e-6, y1, w1, None, w1)),
+                 ("activation x token embedding", side * 6,
+                  lambda: AC.act_mul_embed(u, "gelu_tanh", ids, tab, side, side, side))]
+        for label, nbytes, fn in cases:
+            t = _time(fn)
+            rows.append({"kernel": label, "width": W, "rows": Tn, "ms": t * 1e3,
+                         "GBps": Tn * nbytes / t / 1e9})
+    for r in rows:
+        print(json.dumps(r), flush=True)
     print(json.dumps({"metric": "design_kernel_rates", "rows": rows}), flush=True)
     return 0

@@ -211,10 +211,11 @@ def residual_rms_step(x: torch.Tensor, eps: float, ys=(), w_next: Optional[torch
     if use_hip(x) and W % 4:
         # the kernel sums partials in 16-byte units; other widths (no GEMM of the framework
         # produces them) join the stream through the unfused fp32 sum
-        odd = [(y, g) for y, g in pairs if isinstance(y, SplitK) or isinstance(g, SplitKSlice)]
-        for y, g in odd:
-            x += joined(y, g)
-        pairs = [p for p in pairs if not any(p is o for o in odd)]
+        odd = lambda y, g: isinstance(y, SplitK) or isinstance(g, SplitKSlice)
+        for y, g in pairs:
+            if odd(y, g):
+                x += joined(y, g)
+        pairs = [(y, g) for y, g in pairs if not odd(y, g)]
     if not use_hip(x):
         for y, g in pairs:
             x += joined(y, g)
