@@ -39,8 +39,10 @@ struct HmArgs {
   float* ml;                        // [rows, nparts, H, 2]: its running (max, sum)
 };
 
+typedef __attribute__((ext_vector_type(4))) unsigned int u32x4;
 constexpr float HM_LOG2E = 1.4426950408889634f;
 constexpr int HM_PAGES = 256;       // block -> page entries kept in LDS
+constexpr int HM_QB = 32;           // queries per prefill work item
 
 EIA_DEV float hm_softcap(float s, float cap, float icap2) {
   return cap - 2.f * cap * __builtin_amdgcn_rcpf(exp2f(s * icap2) + 1.f);
@@ -54,152 +56,221 @@ EIA_DEV HmBlocks hm_blocks(int pos_first, int pos_last, int window) {
 EIA_DEV int hm_parts(int nparts, int nblocks) { return min(nparts, max(1, (nblocks + 7) >> 3)); }
 
 // ---------------------------------------------------------------------------------------------
-// Prefill: a wave owns one head of a 16-query tile and NR kv heads' values (grid.z: the subset of
-// kv heads); columns of its tiles are the queries.
-template <int NR, int ND, int NDV>
+// Prefill: a workgroup of four waves (four heads) owns a tile of 32 queries and NR kv heads'
+// values (grid.z: the subset of kv heads); a wave owns one head and both 16-query halves, so
+// every operand it reads feeds two (keys) or four (values: high part and remainder) products.
+// The block's keys (NK distinct kv heads among the four heads) and values are staged in LDS,
+// double buffered: the next block's global loads are in flight during this block's products.
+// LDS rows are swizzled in 16-byte chunks so that the 16 lanes of an operand row group touch
+// different banks.
+template <int NK, int NR, int ND, int NDV>
+struct HmStage {
+  static constexpr int KC = ND * 4;                  // 16-byte chunks of a key row
+  static constexpr int KCH = 32 * KC;                // chunks of one kv head's keys
+  static constexpr int VCH = NDV * 16 * 4;           // chunks of one kv head's values
+  static constexpr int TOT = NK * KCH + NR * VCH;    // chunks of one buffer
+  static constexpr int PT = (TOT + 255) / 256;       // chunks per thread
+};
+// position of chunk j of a key row: 16 rows of one operand tile (rows 8 (c >> 2) + (c & 3) [+ 4])
+// at the same chunk land in 16 different 16-byte columns of the banks
+template <int ND> EIA_DEV int hm_kswz(int row, int j) {
+  const int f = (row & 3) | ((row >> 3) << 2);
+  return ND == 4 ? (j ^ f) : (j ^ (f >> 1));
+}
+EIA_DEV int hm_vswz(int row, int j) { return j ^ ((row >> 2) & 3); }
+
+template <int NK, int NR, int ND, int NDV>
 __global__ void __launch_bounds__(256, 2)
 head_mix_prefill_kernel(const HmArgs a) {
-  const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
+  using S = HmStage<NK, NR, ND, NDV>;
+  extern __shared__ u32x4 stage[];                   // [2][S::TOT]
+  __shared__ int page_s[HM_PAGES];
+  const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int c = lane & 15, g = lane >> 4;
   const int H = a.H, G = a.G, D = a.D, Dv = a.Dv, bs = a.bs, rep = H / G;
   const int nd = (D + 31) >> 5, ndv = Dv >> 4;
   const long krow = (long)G * D, vpage = (long)G * Dv * bs;
   const int seq = a.work[2 * blockIdx.x], q0 = a.work[2 * blockIdx.x + 1];
-  const int row0 = a.cu[seq] + q0, nq = min(16, a.cu[seq + 1] - row0);
-  const int h = blockIdx.y * 4 + wave;
+  const int row0 = a.cu[seq] + q0, nq = min(HM_QB, a.cu[seq + 1] - row0);
+  const int hw0 = blockIdx.y * 4, h = hw0 + wave;
   const bool on = h < H;
-  const int hs = on ? h : 0, kvh = hs / rep;
+  const int hs = on ? h : H - 1;
   const int r0v = blockIdx.z * NR;
   const int* bt = a.bt + (long)seq * a.ldbt;
-  const bool row_ok = c < nq;
-  const long row = row0 + (row_ok ? c : 0);
-  const int qpos = a.positions[row];
-  const HmBlocks kb = hm_blocks(a.positions[row0], a.positions[row0 + nq - 1], a.window);
-  __shared__ int page_s[HM_PAGES];
-  for (int i = threadIdx.x; i < min(kb.n, HM_PAGES); i += blockDim.x)
-    page_s[i] = bt[((kb.b0 + i) << 5) / bs];
-  __syncthreads();
-  if (!on) return;
+  const int pos_first = a.positions[row0], pos_last = a.positions[row0 + nq - 1];
+  const HmBlocks kb = hm_blocks(pos_first, pos_last, a.window);
+  for (int i = tid; i < min(kb.n, HM_PAGES); i += 256) page_s[i] = bt[((kb.b0 + i) << 5) / bs];
   const bf16x8 zero8 = {0, 0, 0, 0, 0, 0, 0, 0};
-  bf16x8 qf[ND];
+  bool row_ok[2];
+  long row[2];
+  int qpos[2];
+  bf16x8 qf[2][ND];
 #pragma unroll
-  for (int s = 0; s < ND; ++s) {
-    const int d = 32 * s + 8 * g;
-    const bf16x8 v = *reinterpret_cast<const bf16x8*>(a.q + row * a.ldq + (long)hs * D + (d < D ? d : 0));
-    qf[s] = d < D ? v : zero8;
-  }
-  const float mult = a.mult[hs], cap = a.cap, icap2 = cap > 0.f ? 2.f * HM_LOG2E / cap : 0.f;
-  f32x4 acc[NR][NDV];
-#pragma unroll
-  for (int r = 0; r < NR; ++r)
-#pragma unroll
-    for (int t = 0; t < NDV; ++t) acc[r][t] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float mrun = -1e30f, lrun = 0.f;
-  const int kr0 = 8 * (c >> 2) + (c & 3);            // key of row c in tile 0 (tile 1: + 4)
-  const int dq = 8 * g;
-  auto load_k = [&](int b, bf16x8 (&kf)[2][ND]) {
-    const int key0 = (kb.b0 + b) << 5;
-    const long page = b < HM_PAGES ? page_s[b] : bt[key0 / bs];
-    const bf16_t* kp = a.kc + (page * bs + key0 % bs + kr0) * krow + (long)kvh * D;
+  for (int u = 0; u < 2; ++u) {
+    row_ok[u] = 16 * u + c < nq;
+    row[u] = row0 + (row_ok[u] ? 16 * u + c : 0);
+    qpos[u] = a.positions[row[u]];
 #pragma unroll
     for (int s = 0; s < ND; ++s) {
-      const int d = 32 * s + dq;
-      const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(kp + (d < D ? d : 0));
-      const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(kp + 4 * krow + (d < D ? d : 0));
-      kf[0][s] = d < D ? k0 : zero8;
-      kf[1][s] = d < D ? k1 : zero8;
+      const int d = 32 * s + 8 * g;
+      const bf16x8 v = *reinterpret_cast<const bf16x8*>(a.q + row[u] * a.ldq + (long)hs * D +
+                                                        (d < D ? d : 0));
+      qf[u][s] = d < D ? v : zero8;
     }
-  };
-  bf16x8 kf[2][ND];
-  load_k(0, kf);
-  for (int b = 0; b < kb.n; ++b) {
+  }
+  const float mult = a.mult[hs], cap = a.cap, icap2 = cap > 0.f ? 2.f * HM_LOG2E / cap : 0.f;
+  f32x4 acc[2][NR][NDV];
+  float mrun[2], lrun[2];
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    mrun[u] = -1e30f;
+    lrun[u] = 0.f;
+#pragma unroll
+    for (int r = 0; r < NR; ++r)
+#pragma unroll
+      for (int t = 0; t < NDV; ++t) acc[u][r][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+  // this thread's chunks of a block: source offsets (elements from the block's first key / value
+  // column) and LDS positions do not change from block to block
+  // (KCH is a multiple of 256, so a thread's p-th chunk is a key chunk for all threads or none)
+  int src[S::PT], dst[S::PT];
+#pragma unroll
+  for (int p = 0; p < S::PT; ++p) {
+    const int x = tid + 256 * p;
+    if (256 * p < NK * S::KCH) {
+      const int k = x / S::KCH, y = x % S::KCH, r = y / S::KC, j = y % S::KC;
+      const int kvh = min(hw0 + k * (4 / NK), H - 1) / rep;
+      src[p] = r * G * D + kvh * D + (8 * j < D ? 8 * j : 0);
+      dst[p] = k * S::KCH + r * S::KC + hm_kswz<ND>(r, j);
+    } else {
+      const int z = min(x, S::TOT - 1) - NK * S::KCH;
+      const int rv = z / S::VCH, y = z % S::VCH, r = y >> 2, j = y & 3;
+      src[p] = (min(r0v + rv, G - 1) * Dv + min(r, Dv - 1)) * bs + 8 * j;
+      dst[p] = NK * S::KCH + rv * S::VCH + r * 4 + hm_vswz(r, j);
+    }
+  }
+  u32x4 stg[S::PT];
+  auto fetch = [&](int b) {
     const int key0 = (kb.b0 + b) << 5;
     const long page = b < HM_PAGES ? page_s[b] : bt[key0 / bs];
-    const bf16_t* vp0 = a.vc + page * vpage + (long)c * bs + key0 % bs + dq;
-    f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
+    const bf16_t* kp = a.kc + (page * bs + key0 % bs) * krow;
+    const bf16_t* vp = a.vc + page * vpage + key0 % bs;
+#pragma unroll
+    for (int p = 0; p < S::PT; ++p)
+      stg[p] = *reinterpret_cast<const u32x4*>((256 * p < NK * S::KCH ? kp : vp) + src[p]);
+  };
+  auto put = [&](int buf) {
+#pragma unroll
+    for (int p = 0; p < S::PT; ++p)
+      if (S::TOT % 256 == 0 || tid + 256 * p < S::TOT) stage[buf * S::TOT + dst[p]] = stg[p];
+  };
+  __syncthreads();                                   // page_s
+  fetch(0);
+  put(0);
+  __syncthreads();
+  const int kr0 = 8 * (c >> 2) + (c & 3);            // key of row c in tile 0 (tile 1: + 4)
+  const int kslot = wave / (4 / NK);
+  for (int b = 0; b < kb.n; ++b) {
+    if (b + 1 < kb.n) fetch(b + 1);
+    const u32x4* K = stage + (b & 1) * S::TOT + kslot * S::KCH;
+    const u32x4* V = stage + (b & 1) * S::TOT + NK * S::KCH;
+    const int key0 = (kb.b0 + b) << 5;
+    f32x4 sc[2][2];
+#pragma unroll
+    for (int u = 0; u < 2; ++u) sc[u][0] = sc[u][1] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int s = 0; s < ND; ++s)
       if (s < nd) {
-        s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[0][s], qf[s], s0, 0, 0, 0);
-        s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[1][s], qf[s], s1, 0, 0, 0);
-      }
-    // the first kv head's values are requested before the softmax arithmetic needs them
-    bf16x8 vf[NDV];
-    {
-      const bf16_t* vp = vp0 + (long)(r0v < G ? r0v : 0) * Dv * bs;
+        const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(
+            K + kr0 * S::KC + hm_kswz<ND>(kr0, 4 * s + g));
+        const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(
+            K + (kr0 + 4) * S::KC + hm_kswz<ND>(kr0 + 4, 4 * s + g));
 #pragma unroll
-      for (int t = 0; t < NDV; ++t)
-        vf[t] = *reinterpret_cast<const bf16x8*>(vp + (long)(t < ndv ? t : 0) * 16 * bs);
-    }
-    if (b + 1 < kb.n) load_k(b + 1, kf);
-    float v[8];
-    bool vis[8];
-    float mloc = -1e30f;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      float s = (e < 4 ? s0[e] : s1[e - 4]) * mult;
-      if (cap > 0.f) s = hm_softcap(s, cap, icap2);
-      const int key = key0 + 8 * g + e;
-      vis[e] = row_ok && key <= qpos && (a.window <= 0 || qpos - key < a.window);
-      v[e] = s;
-      if (vis[e]) mloc = fmaxf(mloc, s);
-    }
-    mloc = fmaxf(mloc, __shfl_xor(mloc, 16, 64));
-    mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64));
-    const float mnew = fmaxf(mrun, mloc);
-    const float alpha = exp2f((mrun - mnew) * HM_LOG2E);
-    bf16x8 ph, pl;
-    float psum = 0.f;
-#pragma unroll
-    for (int e = 0; e < 8; ++e) {
-      const float p = vis[e] ? exp2f((v[e] - mnew) * HM_LOG2E) : 0.f;
-      const bf16_t hi = f2bf(p);
-      ph[e] = hi;
-      pl[e] = f2bf(p - bf2f(hi));
-      psum += p;
-    }
-    psum += __shfl_xor(psum, 16, 64);
-    psum += __shfl_xor(psum, 32, 64);
-    lrun = lrun * alpha + psum;
-    mrun = mnew;
-    const bool resc = __any(alpha != 1.f);            // (uniform)
-#pragma unroll
-    for (int r = 0; r < NR; ++r) {
-      bf16x8 vn[NDV];
-      if (r + 1 < NR) {
-        const bf16_t* vp = vp0 + (long)(r0v + r + 1 < G ? r0v + r + 1 : 0) * Dv * bs;
-#pragma unroll
-        for (int t = 0; t < NDV; ++t)
-          vn[t] = *reinterpret_cast<const bf16x8*>(vp + (long)(t < ndv ? t : 0) * 16 * bs);
-      }
-#pragma unroll
-      for (int t = 0; t < NDV; ++t) {
-        if (t < ndv) {
-          f32x4 o = acc[r][t];
-          if (resc) o *= alpha;
-          o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[t], ph, o, 0, 0, 0);
-          acc[r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[t], pl, o, 0, 0, 0);
+        for (int u = 0; u < 2; ++u) {
+          sc[u][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, qf[u][s], sc[u][0], 0, 0, 0);
+          sc[u][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, qf[u][s], sc[u][1], 0, 0, 0);
         }
       }
-      if (r + 1 < NR) {
+    // a block that every query of the tile sees whole needs no mask
+    const bool whole = nq == HM_QB && key0 + 31 <= pos_first &&
+                       (a.window <= 0 || pos_last - key0 < a.window);
+    bf16x8 ph[2], pl[2];
+    float alpha[2];
 #pragma unroll
-        for (int t = 0; t < NDV; ++t) vf[t] = vn[t];
+    for (int u = 0; u < 2; ++u) {
+      float v[8];
+      float mloc = -1e30f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        float s = sc[u][e >> 2][e & 3] * mult;
+        if (cap > 0.f) s = hm_softcap(s, cap, icap2);
+        if (!whole) {
+          const int key = key0 + 8 * g + e;
+          const bool vis = row_ok[u] && key <= qpos[u] && (a.window <= 0 || qpos[u] - key < a.window);
+          s = vis ? s : -INFINITY;
+        }
+        v[e] = s;
+        mloc = fmaxf(mloc, s);
       }
+      mloc = fmaxf(mloc, __shfl_xor(mloc, 16, 64));
+      mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64));
+      const float mnew = fmaxf(mrun[u], mloc);
+      alpha[u] = exp2f((mrun[u] - mnew) * HM_LOG2E);
+      float psum = 0.f;
+#pragma unroll
+      for (int e = 0; e < 8; ++e) {
+        const float p = exp2f((v[e] - mnew) * HM_LOG2E);
+        const bf16_t hi = f2bf(p);
+        ph[u][e] = hi;
+        pl[u][e] = f2bf(p - bf2f(hi));
+        psum += p;
+      }
+      psum += __shfl_xor(psum, 16, 64);
+      psum += __shfl_xor(psum, 32, 64);
+      lrun[u] = lrun[u] * alpha[u] + psum;
+      mrun[u] = mnew;
     }
-  }
-  if (!row_ok) return;
-  // this lane holds, per kv head and tile t, value columns 16 t + 4 g + i of query c
-  if (blockIdx.z == 0 && g == 0) {
-    a.ml[(row * H + h) * 2] = mrun;
-    a.ml[(row * H + h) * 2 + 1] = lrun;
-  }
+    if (__any(alpha[0] != 1.f || alpha[1] != 1.f)) {
 #pragma unroll
-  for (int r = 0; r < NR; ++r) {
-    if (r0v + r >= G) break;
-    float* dst = a.acc + ((row * H + h) * G + r0v + r) * Dv + 4 * g;
+      for (int u = 0; u < 2; ++u)
 #pragma unroll
-    for (int t = 0; t < NDV; ++t)
-      if (t < ndv) *reinterpret_cast<f32x4*>(dst + 16 * t) = acc[r][t];
+        for (int r = 0; r < NR; ++r)
+#pragma unroll
+          for (int t = 0; t < NDV; ++t) acc[u][r][t] *= alpha[u];
+    }
+#pragma unroll
+    for (int r = 0; r < NR; ++r)
+#pragma unroll
+      for (int t = 0; t < NDV; ++t)
+        if (t < ndv) {
+          const bf16x8 vf = *reinterpret_cast<const bf16x8*>(V + r * S::VCH + (16 * t + c) * 4 +
+                                                             hm_vswz(16 * t + c, g));
+#pragma unroll
+          for (int u = 0; u < 2; ++u) {
+            acc[u][r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[u], acc[u][r][t], 0, 0, 0);
+            acc[u][r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[u], acc[u][r][t], 0, 0, 0);
+          }
+        }
+    if (b + 1 < kb.n) put((b + 1) & 1);              // (its last readers passed the barrier below)
+    __syncthreads();
+  }
+  if (!on) return;
+  // this lane holds, per kv head and tile t, value columns 16 t + 4 g + i of queries c, 16 + c
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    if (!row_ok[u]) continue;
+    if (blockIdx.z == 0 && g == 0) {
+      a.ml[(row[u] * H + h) * 2] = mrun[u];
+      a.ml[(row[u] * H + h) * 2 + 1] = lrun[u];
+    }
+#pragma unroll
+    for (int r = 0; r < NR; ++r) {
+      if (r0v + r >= G) break;
+      float* o = a.acc + ((row[u] * H + h) * G + r0v + r) * Dv + 4 * g;
+#pragma unroll
+      for (int t = 0; t < NDV; ++t)
+        if (t < ndv) *reinterpret_cast<f32x4*>(o + 16 * t) = acc[u][r][t];
+    }
   }
 }
 
@@ -466,10 +537,26 @@ EIA_API int eia_head_mix_attn(const void* q, long ldq, const void* kc, const voi
     else L(NR, 2, 4);                                                                           \
   } while (0)
   if (cu) {
+    // distinct kv heads among the four heads of a workgroup: 1, 2 or (any grouping) one per head
+    const int rep = H / G, nk = rep % 4 == 0 ? 1 : rep % 2 == 0 ? 2 : 4;
+#define HM_PRE1(NK, NR, ND_, NV_)                                                               \
+  do {                                                                                          \
+    constexpr int lds = 2 * HmStage<NK, NR, ND_, NV_>::TOT * 16;                                \
+    if (lds > 48 * 1024)                                                                        \
+      (void)hipFuncSetAttribute(                                                                \
+          reinterpret_cast<const void*>(&head_mix_prefill_kernel<NK, NR, ND_, NV_>),            \
+          hipFuncAttributeMaxDynamicSharedMemorySize, lds);                                     \
+    hipLaunchKernelGGL((head_mix_prefill_kernel<NK, NR, ND_, NV_>),                             \
+                       dim3(n_items, (H + 3) / 4, (G + NR - 1) / NR), dim3(256), lds, st, a);   \
+  } while (0)
 #define HM_PRE(NR, ND_, NV_)                                                                    \
-  hipLaunchKernelGGL((head_mix_prefill_kernel<NR, ND_, NV_>),                                   \
-                     dim3(n_items, (H + 3) / 4, (G + NR - 1) / NR), dim3(256), 0, st, a)
+  do {                                                                                          \
+    if (nk == 1) HM_PRE1(1, NR, ND_, NV_);                                                      \
+    else if (nk == 2) HM_PRE1(2, NR, ND_, NV_);                                                 \
+    else HM_PRE1(4, NR, ND_, NV_);                                                              \
+  } while (0)
     if (G == 1) HM_SIZES(HM_PRE, 1); else HM_SIZES(HM_PRE, 2);
+#undef HM_PRE1
 #undef HM_PRE
   } else {
 #define HM_DEC(NR, ND_, NV_)                                                                    \

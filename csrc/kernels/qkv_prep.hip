@@ -4,7 +4,7 @@
 //
 // Per token row (position p) and channel c of q, k or v (u: the projection, rounded to the
 // activation type):
-//   conv    y_p = sum_j w[c, j] u_(p - taps + 1 + j)     (taps 1 without weights: y = u); zeros
+//   conv    y_p = sum_j w[c, j] u_(p - taps + 1 + j)     (no weights: y = u); zeros
 //           before the sequence's start; earlier tokens of the sequence that are not in this step
 //           come from its state slot, which holds the last taps - 1 projected values
 //   rotate  (q, k) the first rot_dims entries of every head turn by the position: pairs
@@ -157,6 +157,17 @@ qkv_prep_kernel(const QkvPrepArgs a) {
         }
         ua[e][i] = ya;
         ub[e][i] = yb;
+      }
+    }
+  } else if (cw) {                                     // one tap: a factor per channel
+#pragma unroll
+    for (int e = 0; e < NE; ++e) {
+      const float wa = oka[e] ? ld_f32<T>(cw, c0 + da[e]) : 0.f;
+      const float wb = okb[e] ? ld_f32<T>(cw, c0 + db[e]) : 0.f;
+#pragma unroll
+      for (int i = 0; i < QP_ROWS; ++i) {
+        ua[e][i] *= wa;
+        ub[e][i] *= wb;
       }
     }
   }

@@ -106,7 +106,7 @@ class BorosunLayer(nn.Module):
                 H, G, D, Dv, float(m.get("scale", D ** -0.5)),
                 int(rot.get("dims", D if rot else 0)), float(rot.get("base", 10000.0)),
                 rot.get("scaling"), eps, dtype, device, offsets=self.proj.offsets,
-                taps=int(m.get("conv") or 1), qk_norm=second,
+                taps=int(m.get("conv") or 0), qk_norm=second,
                 softcap=float(m.get("softcap") or 0.0),
                 window=int((m.get("mask") or {}).get("size", 0)), head_mix=not second,
                 v_mix=v_mix)

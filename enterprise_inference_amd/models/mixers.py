@@ -740,7 +740,7 @@ class MixAttentionMixer(_WindowMixerBase):
     """Grouped-query softmax attention over the part of a caller's fused projection that holds q,
     k and v (no biases); the caller owns the projection and the output product.  Options:
 
-    * ``taps`` > 1: y_t = sum_j w[c, j] u_(t - taps + 1 + j) on every channel c of q, k and v, zeros
+    * ``taps`` > 0: y_t = sum_j w[c, j] u_(t - taps + 1 + j) on every channel c of q, k and v, zeros
       before the sequence's start (weights ``q_conv`` / ``k_conv`` / ``v_conv`` [channels, taps]);
       a state slot keeps each sequence's last taps - 1 projected values
     * rotation of the first ``rot_dims`` entries of every q / k head (pairs (i, i + rot_dims/2));
@@ -754,13 +754,13 @@ class MixAttentionMixer(_WindowMixerBase):
 
     def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, rot_dims: int,
                  rot_base: float, rot_scaling, eps: float, dtype, device, *, offsets: dict,
-                 taps: int = 1, qk_norm: bool = False, softcap: float = 0.0, window: int = 0,
+                 taps: int = 0, qk_norm: bool = False, softcap: float = 0.0, window: int = 0,
                  head_mix: bool = False, v_mix=None):
         super().__init__()
         if rot_dims > dim or rot_dims % 2:
             raise ValueError("rot.dims must be even and at most dim")
-        if not 1 <= taps <= win_ops.PREP_MAX_TAPS:
-            raise ValueError(f"short convolution: 1 .. {win_ops.PREP_MAX_TAPS} taps")
+        if not 0 <= taps <= win_ops.PREP_MAX_TAPS:
+            raise ValueError(f"short convolution: at most {win_ops.PREP_MAX_TAPS} taps")
         if v_mix not in (None, "first", "later"):
             raise ValueError(f"v_mix {v_mix!r}")
         self._setup(0, heads, kv_heads, dim, vdim, scale, window, 0, eps, [], False, dtype, device,
@@ -768,8 +768,8 @@ class MixAttentionMixer(_WindowMixerBase):
         self.proj = self.proj_bias = None
         self.offsets = {n: offsets[n] for n in ("q", "k", "v")}
         inv_freq, amp = rot_ops.rotary_frequencies(rot_dims, rot_base, rot_scaling, device)
-        self.taps, self.v_mix = int(taps), v_mix
-        conv = lambda n: _plain((n, taps), dtype, device) if taps > 1 else None
+        self.taps, self.v_mix = max(1, int(taps)), v_mix
+        conv = lambda n: _plain((n, taps), dtype, device) if taps else None
         self.q_conv, self.k_conv = conv(heads * dim), conv(kv_heads * dim)
         self.v_conv = conv(kv_heads * vdim)
         self.prep = win_ops.PrepSpec(heads, kv_heads, dim, vdim, inv_freq, int(rot_dims), True, amp,
@@ -797,7 +797,7 @@ class MixAttentionMixer(_WindowMixerBase):
         return (self.taps - 1) * self.prep.channels() * elem
 
     def allocate_state(self, num_slots: int, dtype, device):
-        """[slots, taps - 1, channels] projected values, or None without convolutions."""
+        """[slots, taps - 1, channels] projected values, or None where nothing is kept."""
         if self.taps == 1:
             return None
         return torch.zeros(max(1, num_slots), self.taps - 1, self.prep.channels(), dtype=dtype,

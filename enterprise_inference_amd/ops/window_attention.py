@@ -29,9 +29,11 @@ from typing import List, Optional
 import torch
 
 from ._dispatch import check, lib, ptr, require, stream, use_hip
+from .attention import build_prefill_work
 
 SCALAR_QB = 4            # queries per prefill work item of the scalar-FMA kernel
 MFMA_QB = 16             # ... and of the MFMA kernel (one 16-row tile)
+HEAD_MIX_QB = 32         # ... and of the head-mixing kernel (head_mix_attention.hip HM_QB)
 _MFMA_ENV = os.environ.get("EIA_WINDOW_MFMA", "1") != "0"
 
 
@@ -61,7 +63,8 @@ class WindowSpec:
 
 def build_work(q_lens: List[int], qblock: int) -> List[int]:
     """[seq, first query] pairs; a windowed row's work does not grow with its position, so the
-    order is the batch's own."""
+    order is the batch's own (layers without a window take the longest-first order of
+    ops/attention.py build_prefill_work)."""
     out: List[int] = []
     for s, n in enumerate(q_lens):
         for q0 in range(0, n, qblock):
@@ -120,7 +123,9 @@ def head_mix_partitions(batch: int, spec: WindowSpec, cus: int = 256) -> int:
 
 
 def query_block(spec: WindowSpec, dtype: torch.dtype, block_size: int) -> int:
-    return MFMA_QB if mfma_ok(spec, dtype, block_size) else SCALAR_QB
+    if not mfma_ok(spec, dtype, block_size):
+        return SCALAR_QB
+    return HEAD_MIX_QB if spec.talk_post else MFMA_QB
 
 
 def _rms(v: torch.Tensor, eps: float) -> torch.Tensor:
@@ -285,7 +290,7 @@ class PrepSpec:
     rot_amp: float = 1.0
     norm: bool = False              # every q / k head divided by its root mean square
     eps: float = 0.0
-    taps: int = 1                   # taps of the short convolutions (1: none)
+    taps: int = 1                   # taps of the short convolutions (no weights: none)
     cw_q: Optional[torch.Tensor] = None     # [H*D, taps], [G*D, taps], [G*Dv, taps]
     cw_k: Optional[torch.Tensor] = None
     cw_v: Optional[torch.Tensor] = None
@@ -320,6 +325,8 @@ def _prep_ref(fused, offs, sp: PrepSpec, md, k_cache, v_cache, state, lam, v_fir
                 y[lo:hi] += ext[j:j + hi - lo] * w[:, j]
             state[sl] = ext[-(K - 1):].to(state.dtype)
         u = y
+    elif sp.cw_q is not None:
+        u = u * torch.cat([sp.cw_q, sp.cw_k, sp.cw_v], 0).float()[:, 0]
     q, k, v = torch.split(u, [H * D, G * D, G * Dv], 1)
 
     def side(x, m):
@@ -345,7 +352,7 @@ def qkv_prep_cache(fused, q_off: int, k_off: int, v_off: int, sp: PrepSpec, md,
                    state: Optional[torch.Tensor] = None, lam: Optional[torch.Tensor] = None,
                    v_first: Optional[torch.Tensor] = None, v_mode: int = 0) -> torch.Tensor:
     """From fused projection rows [T, *] to attention inputs: short causal convolution over time
-    on every channel of q, k and v (``sp.taps`` > 1; ``state`` [slots, taps - 1, channels] holds
+    on every channel of q, k and v (``sp.cw_*`` given; with ``sp.taps`` > 1 ``state`` [slots, taps - 1, channels] holds
     each sequence's last projected values), rotation of the first ``sp.rot_dims`` entries of every
     q / k head, an optional weightless RMS norm per head, value mixing, and the cache write.
     ``v_mode`` 1: the values are also stored in ``v_first`` [T, G*Dv]; 2: v <- (1 - lam) v + lam
@@ -379,10 +386,11 @@ def qkv_prep_cache(fused, q_off: int, k_off: int, v_off: int, sp: PrepSpec, md,
             sp.inv_freq.dtype == torch.float32 and sp.inv_freq.numel() >= sp.rot_dims // 2,
             "qkv_prep_cache: rotation")
     require(1 <= sp.taps <= PREP_MAX_TAPS, f"qkv_prep_cache: 1 .. {PREP_MAX_TAPS} taps")
-    if sp.taps > 1:
+    if sp.taps > 1 or sp.cw_q is not None:
         for w, rows in ((sp.cw_q, H * D), (sp.cw_k, G * D), (sp.cw_v, G * Dv)):
             require(w is not None and w.dtype == dt and w.is_contiguous() and
                     w.shape == (rows, sp.taps), "qkv_prep_cache: convolution weights")
+    if sp.taps > 1:
         require(state is not None and state.dtype == dt and state.is_contiguous() and
                 state.shape[1:] == (sp.taps - 1, sp.channels()) and md.seq_slots is not None and
                 md.seq_slots.dtype == torch.int32, "qkv_prep_cache: convolution state")
@@ -554,6 +562,6 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
         launch(0, nd, md.decode_block_tables, md.decode_seq_lens, None, None, 1)
     if md.num_prefill_tokens:
         qb = query_block(spec, q.dtype, bs)
-        work, n_work = md.prefill_work_for(qb, build_work)
+        work, n_work = md.prefill_work_for(qb, build_work if spec.window > 0 else build_prefill_work)
         launch(nd, n_work, md.prefill_block_tables, None, md.prefill_cu_q, work, qb)
     return out
