@@ -88,7 +88,7 @@ head_mix_prefill_kernel(const HmArgs a) {
   const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
   const int c = lane & 15, g = lane >> 4;
   const int H = a.H, G = a.G, D = a.D, Dv = a.Dv, bs = a.bs, rep = H / G;
-  const int nd = (D + 31) >> 5, ndv = Dv >> 4;
+  const int ndv = Dv >> 4;
   const long krow = (long)G * D, vpage = (long)G * Dv * bs;
   const int seq = a.work[2 * blockIdx.x], q0 = a.work[2 * blockIdx.x + 1];
   const int row0 = a.cu[seq] + q0, nq = min(HM_QB, a.cu[seq + 1] - row0);
@@ -150,11 +150,12 @@ head_mix_prefill_kernel(const HmArgs a) {
     }
   }
   u32x4 stg[S::PT];
+  int off = (kb.b0 << 5) % bs;                       // the next block to fetch: place in its page
   auto fetch = [&](int b) {
-    const int key0 = (kb.b0 + b) << 5;
-    const long page = b < HM_PAGES ? page_s[b] : bt[key0 / bs];
-    const bf16_t* kp = a.kc + (page * bs + key0 % bs) * krow;
-    const bf16_t* vp = a.vc + page * vpage + key0 % bs;
+    const long page = b < HM_PAGES ? page_s[b] : bt[((kb.b0 + b) << 5) / bs];
+    const bf16_t* kp = a.kc + (page * bs + off) * krow;
+    const bf16_t* vp = a.vc + page * vpage + off;
+    off = off + 32 == bs ? 0 : off + 32;
 #pragma unroll
     for (int p = 0; p < S::PT; ++p)
       stg[p] = *reinterpret_cast<const u32x4*>((256 * p < NK * S::KCH ? kp : vp) + src[p]);
@@ -179,18 +180,17 @@ head_mix_prefill_kernel(const HmArgs a) {
 #pragma unroll
     for (int u = 0; u < 2; ++u) sc[u][0] = sc[u][1] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-    for (int s = 0; s < ND; ++s)
-      if (s < nd) {
-        const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(
-            K + kr0 * S::KC + hm_kswz<ND>(kr0, 4 * s + g));
-        const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(
-            K + (kr0 + 4) * S::KC + hm_kswz<ND>(kr0 + 4, 4 * s + g));
+    for (int s = 0; s < ND; ++s) {                   // (past D: the query operand is zero)
+      const bf16x8 k0 = *reinterpret_cast<const bf16x8*>(
+          K + kr0 * S::KC + hm_kswz<ND>(kr0, 4 * s + g));
+      const bf16x8 k1 = *reinterpret_cast<const bf16x8*>(
+          K + (kr0 + 4) * S::KC + hm_kswz<ND>(kr0 + 4, 4 * s + g));
 #pragma unroll
-        for (int u = 0; u < 2; ++u) {
-          sc[u][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, qf[u][s], sc[u][0], 0, 0, 0);
-          sc[u][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, qf[u][s], sc[u][1], 0, 0, 0);
-        }
+      for (int u = 0; u < 2; ++u) {
+        sc[u][0] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k0, qf[u][s], sc[u][0], 0, 0, 0);
+        sc[u][1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k1, qf[u][s], sc[u][1], 0, 0, 0);
       }
+    }
     // a block that every query of the tile sees whole needs no mask
     const bool whole = nq == HM_QB && key0 + 31 <= pos_first &&
                        (a.window <= 0 || pos_last - key0 < a.window);
@@ -199,19 +199,23 @@ head_mix_prefill_kernel(const HmArgs a) {
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
       float v[8];
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = sc[u][e >> 2][e & 3] * mult;
+      if (cap > 0.f) {
+#pragma unroll
+        for (int e = 0; e < 8; ++e) v[e] = hm_softcap(v[e], cap, icap2);
+      }
+      if (!whole) {
+        const int far = a.window > 0 ? a.window : 0x7fffffff;
+#pragma unroll
+        for (int e = 0; e < 8; ++e) {
+          const int back = qpos[u] - (key0 + 8 * g + e);
+          v[e] = row_ok[u] && back >= 0 && back < far ? v[e] : -INFINITY;
+        }
+      }
       float mloc = -1e30f;
 #pragma unroll
-      for (int e = 0; e < 8; ++e) {
-        float s = sc[u][e >> 2][e & 3] * mult;
-        if (cap > 0.f) s = hm_softcap(s, cap, icap2);
-        if (!whole) {
-          const int key = key0 + 8 * g + e;
-          const bool vis = row_ok[u] && key <= qpos[u] && (a.window <= 0 || qpos[u] - key < a.window);
-          s = vis ? s : -INFINITY;
-        }
-        v[e] = s;
-        mloc = fmaxf(mloc, s);
-      }
+      for (int e = 0; e < 8; ++e) mloc = fmaxf(mloc, v[e]);
       mloc = fmaxf(mloc, __shfl_xor(mloc, 16, 64));
       mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64));
       const float mnew = fmaxf(mrun[u], mloc);
@@ -241,16 +245,15 @@ head_mix_prefill_kernel(const HmArgs a) {
 #pragma unroll
     for (int r = 0; r < NR; ++r)
 #pragma unroll
-      for (int t = 0; t < NDV; ++t)
-        if (t < ndv) {
-          const bf16x8 vf = *reinterpret_cast<const bf16x8*>(V + r * S::VCH + (16 * t + c) * 4 +
-                                                             hm_vswz(16 * t + c, g));
+      for (int t = 0; t < NDV; ++t) {                // (tiles past Dv: staged repeats, not stored)
+        const bf16x8 vf = *reinterpret_cast<const bf16x8*>(V + r * S::VCH + (16 * t + c) * 4 +
+                                                           hm_vswz(16 * t + c, g));
 #pragma unroll
-          for (int u = 0; u < 2; ++u) {
-            acc[u][r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[u], acc[u][r][t], 0, 0, 0);
-            acc[u][r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[u], acc[u][r][t], 0, 0, 0);
-          }
+        for (int u = 0; u < 2; ++u) {
+          acc[u][r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, ph[u], acc[u][r][t], 0, 0, 0);
+          acc[u][r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, pl[u], acc[u][r][t], 0, 0, 0);
         }
+      }
     if (b + 1 < kb.n) put((b + 1) & 1);              // (its last readers passed the barrier below)
     __syncthreads();
   }
@@ -291,7 +294,7 @@ head_mix_decode_kernel(const HmArgs a) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int c = lane & 15, g = lane >> 4;
   const int H = a.H, G = a.G, D = a.D, Dv = a.Dv, bs = a.bs, rep = H / G;
-  const int nd = (D + 31) >> 5, ndv = Dv >> 4;
+  const int ndv = Dv >> 4;
   const long krow = (long)G * D, vpage = (long)G * Dv * bs;
   const int row = blockIdx.x, z = blockIdx.z;
   const int nsub = (G + NR - 1) / NR;
@@ -362,13 +365,12 @@ head_mix_decode_kernel(const HmArgs a) {
         if (k0 + j <= k_hi) {
           const bool mine = grp == k0 + j;
 #pragma unroll
-          for (int s = 0; s < ND; ++s)
-            if (s < nd) {
-              const bf16x8 qm = mine ? qf[s] : zero8;
-              // (d >= D: the query operand is zero and the key operand a finite repeat)
-              s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j][0][s], qm, s0, 0, 0, 0);
-              s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j][1][s], qm, s1, 0, 0, 0);
-            }
+          for (int s = 0; s < ND; ++s) {
+            const bf16x8 qm = mine ? qf[s] : zero8;
+            // (d >= D: the query operand is zero and the key operand a finite repeat)
+            s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j][0][s], qm, s0, 0, 0, 0);
+            s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j][1][s], qm, s1, 0, 0, 0);
+          }
         }
       }
     }
@@ -378,12 +380,17 @@ head_mix_decode_kernel(const HmArgs a) {
     float mloc = -1e30f;
 #pragma unroll
     for (int e = 0; e < 8; ++e) {
-      float s = (e < 4 ? s0[e] : s1[e - 4]) * mult;
-      if (cap > 0.f) s = hm_softcap(s, cap, icap2);
+      v[e] = (e < 4 ? s0[e] : s1[e - 4]) * mult;
+    }
+    if (cap > 0.f) {
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = hm_softcap(v[e], cap, icap2);
+    }
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
       const int key = key0 + 8 * g + e;
       vis[e] = key <= qpos && (a.window <= 0 || qpos - key < a.window);
-      v[e] = s;
-      if (vis[e]) mloc = fmaxf(mloc, s);
+      mloc = fmaxf(mloc, vis[e] ? v[e] : -1e30f);
     }
     mloc = fmaxf(mloc, __shfl_xor(mloc, 16, 64));
     mloc = fmaxf(mloc, __shfl_xor(mloc, 32, 64));
@@ -406,12 +413,11 @@ head_mix_decode_kernel(const HmArgs a) {
 #pragma unroll
     for (int r = 0; r < NR; ++r)
 #pragma unroll
-      for (int t = 0; t < NDV; ++t)
-        if (t < ndv) {
-          f32x4 o = acc[r][t] * alpha;
-          o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[r][t], ph, o, 0, 0, 0);
-          acc[r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[r][t], pl, o, 0, 0, 0);
-        }
+      for (int t = 0; t < NDV; ++t) {
+        f32x4 o = acc[r][t] * alpha;
+        o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[r][t], ph, o, 0, 0, 0);
+        acc[r][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[r][t], pl, o, 0, 0, 0);
+      }
   }
   // merge the four waves
   if (g == 0) {
@@ -555,7 +561,8 @@ EIA_API int eia_head_mix_attn(const void* q, long ldq, const void* kc, const voi
     else if (nk == 2) HM_PRE1(2, NR, ND_, NV_);                                                 \
     else HM_PRE1(4, NR, ND_, NV_);                                                              \
   } while (0)
-    if (G == 1) HM_SIZES(HM_PRE, 1); else HM_SIZES(HM_PRE, 2);
+    // (one kv head's values at a time where two do not fit the registers)
+    if (G == 1 || (nk == 4 && bk && bv)) HM_SIZES(HM_PRE, 1); else HM_SIZES(HM_PRE, 2);
 #undef HM_PRE1
 #undef HM_PRE
   } else {

@@ -527,7 +527,7 @@ window_attn_mfma_kernel(const WinAttnArgs a) {
   const int lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
   const int c = lane & 15, g = lane >> 4;
   const int H = a.H, D = a.D, Dv = a.Dv, M = H * P, rep = H / a.G, bs = a.bs;
-  const int nd = (D + 31) >> 5, ndv = Dv >> 4;
+  const int ndv = Dv >> 4;
   const bf16_t* q = (const bf16_t*)a.q;
   const bf16_t* kc = (const bf16_t*)a.kc;
   const bf16_t* vc = (const bf16_t*)a.vc;
@@ -687,11 +687,9 @@ window_attn_mfma_kernel(const WinAttnArgs a) {
           const int m = (j * HPK + hh) * P + pm;
           f32x4 s0 = {0.f, 0.f, 0.f, 0.f}, s1 = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-          for (int s = 0; s < ND; ++s) {
-            if (s < nd) {
-              s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j][pm][0][s], qf[m][s], s0, 0, 0, 0);
-              s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j][pm][1][s], qf[m][s], s1, 0, 0, 0);
-            }
+          for (int s = 0; s < ND; ++s) {             // (past D both operands are zero)
+            s0 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j][pm][0][s], qf[m][s], s0, 0, 0, 0);
+            s1 = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf[j][pm][1][s], qf[m][s], s1, 0, 0, 0);
           }
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
@@ -812,12 +810,10 @@ window_attn_mfma_kernel(const WinAttnArgs a) {
     for (int m = 0; m < MW; ++m) {
       const int j = (m / P) / HPK;
 #pragma unroll
-      for (int t = 0; t < NDV; ++t) {
-        if (t < ndv) {
-          f32x4 o = SIG ? acc[m][t] : acc[m][t] * alpha[m];
-          o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[j][t], ph[m], o, 0, 0, 0);
-          acc[m][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[j][t], pl[m], o, 0, 0, 0);
-        }
+      for (int t = 0; t < NDV; ++t) {                // (tiles past Dv repeat tile 0, not stored;
+        f32x4 o = SIG ? acc[m][t] : acc[m][t] * alpha[m];       // a branch per tile costs more)
+        o = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[j][t], ph[m], o, 0, 0, 0);
+        acc[m][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[j][t], pl[m], o, 0, 0, 0);
       }
     }
   }
