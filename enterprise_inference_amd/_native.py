@@ -105,6 +105,8 @@ _SIGNATURES = {
     "eia_post_rms": [P, L, P, I, P, P, P, P, P, L, F, I, I, I, S],
     "eia_act_mul_embed": [P, L, P, I, L, IP, P, L, I, I, P, I, I, I, I, I, S],
     "eia_softcap": [P, L, F, S],
+    "eia_token_side": [P, P, L, P, L, P, L, P, L, IP, P, L, I, I, P, P, P, P, P, L, F, I, I, I, I, S],
+    "eia_token_side_ok": [I, I],
     "eia_xielu": [P, L, P, I, L, P, P, L, I, I, I, S],
     "eia_sigmoid_gate": [P, L, L, I, P, L, P, L, I, I, I, S],
     "eia_window_attn_mfma_ok": [I, I, I, I, I, I, I],

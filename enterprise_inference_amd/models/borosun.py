@@ -23,9 +23,10 @@ l<i>.side.gate|proj|norm.
 Residual stream, norms, angles, scores, softmax weights and their mixing, decays and the recurrent
 state are fp32 whatever the activation dtype; with dtype float32 the matrix products are fp32 too.
 Everything that reads h rides in one fused projection (mixer inputs and both gates) and one gated
-feed-forward GEMM; a layer's end is four launches (gated residual sum, side gate GEMM, activation
-times token embedding, side projection GEMM) plus one that adds the normed side output and forms
-the next layer's input.
+feed-forward GEMM.  A layer's end is one launch for prompt-sized batches (ops/norm.py
+token_side_step); decode-sized ones take five (gated residual sum, side gate GEMM, activation
+times token embedding, side projection GEMM, and the normed side output with the next layer's
+input norm).
 """
 
 from __future__ import annotations
@@ -67,6 +68,15 @@ class TokenSide(nn.Module):
         self.gate.weight_loader = lambda p, t, sid=None: p.data[:dim].copy_(t)
         self.proj.weight_loader = lambda p, t, sid=None: p.data[:, :dim].copy_(t)
         self.norm = _plain((width,), dtype, device)
+        # copies in matrix-core operand order for the prompt-sized form (refreshed IN PLACE)
+        self.packed = None
+        if dtype == torch.bfloat16 and width % 32 == 0:
+            self.packed = [torch.zeros_like(p.data) for p in (self.gate, self.proj)]
+
+    def refresh(self) -> None:
+        if self.packed is not None:
+            for dst, w in zip(self.packed, (self.gate, self.proj)):
+                dst.copy_(norm_ops.pack_operand(w.data))
 
     def forward(self, xb: torch.Tensor, ids: torch.Tensor, table: torch.Tensor):
         """xb: the residual in the activation dtype -> y (a tensor or gemm.SplitK)."""
@@ -135,9 +145,13 @@ class BorosunLayer(nn.Module):
             gates.append(gemm.columns(fused, *self.proj.offsets["rg2"]))
         if self.side is None:
             return norm_ops.residual_rms_step(x, self.eps, ys, w_next, gates)
+        s = self.side
+        if s.packed is not None and norm_ops.token_side_ok(x, ys, gates, s.pad, h.dtype):
+            return norm_ops.token_side_step(x, self.eps, ys, gates, ids, table, s.col0, s.dim,
+                                            *s.packed, s.norm, w_next)       # prompt-sized
         xb = norm_ops.residual_rms_step(x, self.eps, ys, None, gates, copy_dtype=h.dtype)
-        y = self.side(xb, ids, table)
-        return norm_ops.group_norm_step(x, 1, self.eps, y, self.side.norm, None, w_next)
+        y = s(xb, ids, table)
+        return norm_ops.group_norm_step(x, 1, self.eps, y, s.norm, None, w_next)
 
 
 class BorosunForCausalLM(nn.Module):
@@ -335,3 +349,5 @@ class BorosunForCausalLM(nn.Module):
     def post_load(self) -> None:
         for L in self.layers:
             L.mix.refresh()
+            if L.side is not None:
+                L.side.refresh()

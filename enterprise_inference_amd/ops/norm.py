@@ -268,6 +268,62 @@ def residual_rms_step(x: torch.Tensor, eps: float, ys=(), w_next: Optional[torch
     return h
 
 
+TOKEN_SIDE_MIN_ROWS = 256     # below it the unfused launches fill the chip better
+
+
+def token_side_ok(x: torch.Tensor, ys, gates, pad: int, dtype) -> bool:
+    """Whether ``token_side_step`` takes this layer end: bf16 on the GPU, a prompt-sized batch of
+    stored (not split-K) rows, a supported width."""
+    T, W = x.shape
+    return (use_hip(x) and dtype == torch.bfloat16 and T >= TOKEN_SIDE_MIN_ROWS and
+            1 <= len(ys) <= 2 and
+            all(isinstance(t, torch.Tensor) and t.stride(-1) == 1 and t.stride(0) % 4 == 0 and
+                t.data_ptr() % 8 == 0 for t in list(ys) + list(gates)) and
+            bool(lib().eia_token_side_ok(W, pad)))
+
+
+def pack_operand(w: torch.Tensor) -> torch.Tensor:
+    """[N, K] row-major -> matrix-core operand order, same shape: [16-row tile][32-column step]
+    [lane r + 16 g][8] (row r of the tile, columns 8 g .. 8 g + 7 of the step)."""
+    N, K = w.shape
+    return w.reshape(N // 16, 16, K // 32, 4, 8).permute(0, 2, 3, 1, 4).contiguous().view(N, K)
+
+
+def token_side_step(x: torch.Tensor, eps: float, ys, gates, ids: torch.Tensor,
+                    table: torch.Tensor, col0: int, n: int, gate_w: torch.Tensor,
+                    proj_w: torch.Tensor, w_side: torch.Tensor,
+                    w_next: Optional[torch.Tensor] = None) -> Optional[torch.Tensor]:
+    """A whole layer end in one launch (csrc/kernels/token_side.hip), x fp32 [T, W] in place:
+
+        x += sum_q y_q * sigmoid(g_q)
+        y  = W_proj (gelu_tanh(W_gate x) * table[ids, col0:col0 + n])
+        x += y / sqrt(mean(y^2) + eps) * w_side
+        h  = x / sqrt(mean(x^2) + eps) * w_next      (w_next given: returned)
+
+    ``gate_w`` [pad, W] and ``proj_w`` [W, pad] are zero past ``n`` and packed by
+    ``pack_operand``.  See ``token_side_ok``."""
+    T, W = x.shape
+    bf = torch.bfloat16
+    pad = gate_w.shape[0]
+    require(x.dtype == torch.float32 and x.is_contiguous() and len(ys) == len(gates) and
+            all(t.shape == (T, W) and t.dtype == bf for t in list(ys) + list(gates)),
+            "token_side_step: rows")
+    require(gate_w.shape == (pad, W) and proj_w.shape == (W, pad) and gate_w.is_contiguous() and
+            proj_w.is_contiguous() and w_side.numel() == W and
+            all(t is None or t.dtype == bf for t in (gate_w, proj_w, w_side, w_next, table)) and
+            table.stride(1) == 1 and 0 < n <= pad and col0 + n <= table.shape[1] and
+            (w_next is None or w_next.numel() == W) and ids.dtype == torch.int32 and
+            ids.numel() >= T, "token_side_step: weights")
+    h = torch.empty(T, W, dtype=bf, device=x.device) if w_next is not None else None
+    y2, g2 = (ys[1], gates[1]) if len(ys) > 1 else (None, None)
+    check(lib().eia_token_side(
+        ptr(x), ptr(ys[0]), ys[0].stride(0), ptr(gates[0]), gates[0].stride(0), ptr(y2),
+        y2.stride(0) if y2 is not None else 0, ptr(g2), g2.stride(0) if g2 is not None else 0,
+        ptr(ids), ptr(table), table.stride(0), col0, table.shape[0], ptr(gate_w), ptr(proj_w),
+        ptr(w_side), ptr(w_next), ptr(h), W, float(eps), T, W, n, pad, stream(x)), "token_side")
+    return h
+
+
 def hyper_step(X: torch.Tensor, eps: float, y=None, mix: Optional[torch.Tensor] = None,
                outw: Optional[torch.Tensor] = None, ymult: float = 1.0,
                in_next: Optional[torch.Tensor] = None, w_next: Optional[torch.Tensor] = None,

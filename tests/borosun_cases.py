@@ -3,6 +3,8 @@ framework's PyTorch ops in fp32, the GPU file on the HIP kernels in fp32 and bf1
 
 from __future__ import annotations
 
+import math
+
 import numpy as np
 import torch
 
@@ -164,6 +166,48 @@ def case_act_mul_embed(device, dtype):
     got = act.softcap_(x.clone().to(device), 7.0)
     assert np.allclose(_np(got), O.softcap(_np(x), 7.0), atol=1e-5)
     assert torch.equal(act.softcap_(x.clone().to(device), 0.0).cpu(), x)
+
+
+def case_token_side(W=256, n=24, T=300, sublayers=2, nxt=True):
+    """The whole layer end in one launch (bf16, prompt-sized): a last workgroup that is partly
+    empty, one or two sublayers, gates as columns of a wider row, side widths below, at and above
+    the padding unit, widths that do not fill the last wave's tiles, with and without a next norm."""
+    from enterprise_inference_amd.ops import norm
+    g = torch.Generator().manual_seed(31)
+    bf = torch.bfloat16
+    rnd = lambda *s, k=1.0: (torch.randn(*s, generator=g) * k)
+    x = rnd(T, W, k=2.0)
+    ys = [rnd(T, W).to(bf) for _ in range(sublayers)]
+    wide = rnd(T, 2 * W + 8).to(bf)
+    pad = -(-n // 128) * 128
+    gw, pw = torch.zeros(pad, W), torch.zeros(W, pad)
+    gw[:n], pw[:, :n] = rnd(n, W, k=W ** -0.5), rnd(W, n, k=n ** -0.5)
+    gw, pw = gw.to(bf), pw.to(bf)
+    table = rnd(40, 3 * n).to(bf)
+    ids = torch.randint(0, 40, (T,), generator=g).to(torch.int32)
+    ws, wn = (1 + rnd(W, k=0.2)).to(bf), (1 + rnd(W, k=0.2)).to(bf)
+    xd, wd = x.clone().cuda(), wide.cuda()
+    ysd = [y.cuda() for y in ys]
+    gates = [wd[:, q * W + 8 * q:q * W + 8 * q + W] for q in range(sublayers)]
+    assert norm.token_side_ok(xd, ysd, gates, pad, bf)
+    h = norm.token_side_step(xd, 1e-5, ysd, gates, ids.cuda(), table.cuda(), n, n,
+                             norm.pack_operand(gw.cuda()), norm.pack_operand(pw.cuda()), ws.cuda(), wn.cuda() if nxt else None)
+    want = _np(x)
+    for q in range(sublayers):
+        want = want + _np(ys[q]) * O.sigmoid(_np(wide)[:, q * W + 8 * q:q * W + 8 * q + W])
+    e = _np(table)[ids.long().numpy(), n:2 * n]
+    z = O.gelu_tanh(want @ _np(gw)[:n].T) * e
+    y = z @ _np(pw)[:, :n].T
+    want = want + np.stack([O.rms(r, 1e-5) for r in y]) * _np(ws)
+    # (the products read the residual and the side values in bf16)
+    assert np.allclose(_np(xd), want, atol=5e-2, rtol=1e-2), np.abs(_np(xd) - want).max()
+    d = _np(xd) - want
+    assert math.sqrt(float((d * d).mean())) < 6e-3
+    if nxt:
+        hw = np.stack([O.rms(r, 1e-5) for r in want]) * _np(wn)
+        assert np.allclose(_np(h), hw, atol=3e-2, rtol=2e-2)
+    else:
+        assert h is None
 
 
 def case_prep(device, dtype, H=4, G=2, D=10, Dv=6, dims=6, taps=3, normed=False, T=45, bs=16,
@@ -489,6 +533,30 @@ def case_schedules(device, dtype, cfg_fn=C.config_a, seed=0, block_size=16):
         _check(got2[-1:], want["c"][4:], dtype, "again c")
         bm = sess.scheduler.bm
         assert bm.num_free_blocks() == bm.num_blocks and bm.slots.num_free() == 4
+    finally:
+        sess.close()
+
+
+def case_long_prompt(device, dtype, cfg_fn=C.config_c, n=330, block_size=32):
+    """A prompt long enough for the prompt-sized forms, its first portion beside a decoding
+    request, then a second portion and single tokens: the logits do not depend on which form a
+    row takes."""
+    cfg = cfg_fn()
+    W = _weights(cfg, 4, dtype)
+    t, o = _tokens(n, cfg["vocab"], 41), _tokens(9, cfg["vocab"], 42)
+    want, want_o = C.oracle_logits(cfg, W, t), C.oracle_logits(cfg, W, o)
+    sess = C.make_session(cfg, W, device, dtype, max_tokens=384, block_size=block_size, max_live=2)
+    try:
+        e = lambda k, s, lo, hi: {"id": k, "tokens": s[lo:hi], "want": list(range(hi - lo))}
+        got, got_o = [], [sess.step([e("o", o, 0, 8)])]
+        out = sess.step([e("o", o, 8, 9), e("x", t, 0, 300)], end=["o"])
+        got_o.append(out[:1])
+        got.append(out[1:])
+        got.append(sess.step([e("x", t, 300, 325)]))
+        for i in range(325, n):
+            got.append(sess.step([e("x", t, i, i + 1)]))
+        _check(torch.cat(got), want, dtype, "long prompt")
+        _check(torch.cat(got_o), want_o, dtype, "beside it")
     finally:
         sess.close()
 

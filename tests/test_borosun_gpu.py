@@ -19,6 +19,18 @@ def test_kernel(case, dtype):
     case("cuda", dtype)
 
 
+@pytest.mark.parametrize("shape", [(256, 24, 300, 2, True), (64, 128, 257, 1, False),
+                                   (1056, 130, 256, 2, True), (2048, 256, 270, 2, True),
+                                   (480, 500, 256, 1, True)], ids=lambda s: "-".join(map(str, s)))
+def test_token_side(shape):
+    K.case_token_side(*shape)
+
+
+@pytest.mark.parametrize("cfg", [C.config_c, C.config_d], ids=lambda f: f.__name__)
+def test_long_prompt_mixed_with_decoding(cfg):
+    K.case_long_prompt("cuda", torch.bfloat16, cfg)
+
+
 @pytest.mark.parametrize("dtype", DTYPES, ids=IDS)
 @pytest.mark.parametrize("shape", [
     # H, G, D, Dv, rotated entries, taps, head norm, page, split-K partials
