@@ -894,7 +894,7 @@ def borosun_kernel_rates(a) -> int:
         del kcd, vcd
     # ---- scans
     for Hh, Dk, Dv in ((32, 64, 64), (16, 64, 128), (16, 128, 128)):
-        for nseq, per in ((1, 4096), (4, 2048), (64, 1)):
+        for nseq, per in ((1, 4096), (4, 2048), (16, 128), (64, 1)):
             Tn = nseq * per
             slots = torch.arange(nseq, dtype=torch.int32, device=dev)
             cu = torch.arange(0, Tn + 1, per, dtype=torch.int32, device=dev)
@@ -958,6 +958,20 @@ def borosun_kernel_rates(a) -> int:
                   lambda: N.group_norm_step(x, 4, 1e-6, y1, w1, None, w1)),
                  ("activation x token embedding", side * 6,
                   lambda: AC.act_mul_embed(u, "gelu_tanh", ids, tab, side, side, side))]
+        gw, pw = torch.randn(side, W, device=dev).to(bf) * 0.03, torch.randn(W, side, device=dev).to(bf) * 0.1
+        gp, pp = N.pack_operand(gw), N.pack_operand(pw)
+        gates = (gt[:, :W], gt[:, W:])
+
+        def chain():
+            xb = N.residual_rms_step(x, 1e-6, (y1, y2), None, gates, copy_dtype=bf)
+            g_ = AC.act_mul_embed(torch.nn.functional.linear(xb, gw), "gelu_tanh", ids, tab, side,
+                                  side, side)
+            N.group_norm_step(x, 1, 1e-6, torch.nn.functional.linear(g_, pw), w1, None, w1)
+        # (bytes: the residual once in and out, both outputs and gates in, the next input out)
+        cases += [("layer end, one launch", W * (8 + 4 * 2 + 2),
+                   lambda: N.token_side_step(x, 1e-6, (y1, y2), gates, ids, tab, side, side, gp, pp,
+                                             w1, w1)),
+                  ("layer end, five launches", W * (8 + 4 * 2 + 2), chain)]
         for label, nbytes, fn in cases:
             t = _time(fn)
             rows.append({"kernel": label, "width": W, "rows": Tn, "ms": t * 1e3,
