@@ -21,8 +21,9 @@
 //
 // q, k, v, the gate and the gate pre-activations are column ranges of one fused projection row
 // per token (type T: bf16 or float).  Decays, gates, exponentials, the state, the normaliser and
-// the head norm are fp32, as is mode 2's last decay product.  A sequence whose first row of the step is position 0 starts from the
-// initial state whatever its slot held, so slots are reused without clearing.
+// the head norm are fp32, as is mode 2's last decay product.  A sequence whose first row of the
+// step is position 0 starts from the initial state whatever its slot held, so slots are reused
+// without clearing.
 // Batch layout: sequence s owns rows [cu[s], cu[s+1]) (cu == nullptr: row s).
 #include "eia_common.h"
 
@@ -61,8 +62,8 @@ EIA_DEV float ls_chan_log(const ScanArgs& a, const T* xr, int h, int j) {
 // to LDS, the gate recurrence of the chunk runs (its transcendentals in parallel over the
 // tokens, the running maximum serially in one thread), then the state recurrence runs TC steps on
 // LDS broadcasts leaving four partial outputs per token and column, which are summed, divided,
-// normed and gated.  CH: a decay per key channel (mode 2), staged beside k.  NRM: the normaliser n rides along (every thread of a quarter keeps the
-// quarter's rows of n; column 0 reports n . q).
+// normed and gated.  CH: a decay per key channel (mode 2), staged beside k.  NRM: the normaliser n
+// rides along (every thread of a quarter keeps the quarter's rows of n; column 0 reports n . q).
 template <typename T, int DMAX, bool NRM, bool CH>
 __global__ void __launch_bounds__(4 * (DMAX < 64 ? 64 : DMAX))
 linear_scan_kernel(ScanArgs a) {
@@ -254,7 +255,8 @@ EIA_API int eia_linear_scan(const void* x, long ld, int q_off, int k_off, int v_
                             const float* a2t, const float* a2b, float inv_tau, int norm_h,
                             int is_bf16, hipStream_t st) {
   if (nseq < 0 || H < 1 || D < 1 || Dv < 1 || !x || !y || !S || !slots || !positions ||
-      mode < 0 || mode > 2 || (mode == 2 && (R < 1 || !a2t)) || (mode == 0 && !decay) || (mode == 1 && (!N || !M || cap < 0.f)) ||
+      mode < 0 || mode > 2 || (mode == 2 && (R < 1 || !a2t)) || (mode == 0 && !decay) ||
+      (mode == 1 && (!N || !M || cap < 0.f)) ||
       rot_dims < 0 || rot_dims > D || (rot_dims & 1) || (rot_dims && !inv_freq) ||
       (gate_act != 0 && gate_act != 1))
     return EIA_BAD_SHAPE;
@@ -604,31 +606,31 @@ ls_chunk_out_kernel(ScanArgs a, ChunkArgs c) {
       sq[t][j] *= expf(sC[8 * (t >> 3) - 1][j]);
     }
   } else {
-  ls_chunk_decay(a, c, row0, n, h, sA, sB);
-  __syncthreads();
-  // weights of the chunk's own pairs: P[t][u] = (q_t . k_u) exp(A_t - A_u + log b_u), u <= t
-  for (int idx = tid; idx < LC * LC; idx += 256) {
-    const int t = idx / LC, u = idx % LC;
-    float p = 0.f;
-    if (u <= t && t < n) {
-      const f32x4* qa = reinterpret_cast<const f32x4*>(sq[t]);
-      const f32x4* ka = reinterpret_cast<const f32x4*>(sk[u]);
-#pragma unroll 8
-      for (int i = 0; i < LD / 4; ++i) {
-        const f32x4 x = qa[i], y = ka[i];
-        p += x[0] * y[0] + x[1] * y[1] + x[2] * y[2] + x[3] * y[3];
+    ls_chunk_decay(a, c, row0, n, h, sA, sB);
+    __syncthreads();
+    // weights of the chunk's own pairs: P[t][u] = (q_t . k_u) exp(A_t - A_u + log b_u), u <= t
+    for (int idx = tid; idx < LC * LC; idx += 256) {
+      const int t = idx / LC, u = idx % LC;
+      float p = 0.f;
+      if (u <= t && t < n) {
+        const f32x4* qa = reinterpret_cast<const f32x4*>(sq[t]);
+        const f32x4* ka = reinterpret_cast<const f32x4*>(sk[u]);
+  #pragma unroll 8
+        for (int i = 0; i < LD / 4; ++i) {
+          const f32x4 x = qa[i], y = ka[i];
+          p += x[0] * y[0] + x[1] * y[1] + x[2] * y[2] + x[3] * y[3];
+        }
+        p *= expf(sA[t] - sA[u] + sB[u]);
       }
-      p *= expf(sA[t] - sA[u] + sB[u]);
+      P[t][u] = p;
     }
-    P[t][u] = p;
-  }
-  // n_before . q_t of the gated mode
-  if (a.mode == 1 && tid < n) {
-    const float* nb = c.wsN + ((long)ch * a.H + h) * D;
-    float d = 0.f;
-    for (int i = 0; i < D; ++i) d += nb[i] * sq[tid][i];
-    snq[tid] = d;
-  }
+    // n_before . q_t of the gated mode
+    if (a.mode == 1 && tid < n) {
+      const float* nb = c.wsN + ((long)ch * a.H + h) * D;
+      float d = 0.f;
+      for (int i = 0; i < D; ++i) d += nb[i] * sq[tid][i];
+      snq[tid] = d;
+    }
   }
   __syncthreads();
   const int r = tid >> 7, j = tid & 127;

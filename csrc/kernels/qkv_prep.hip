@@ -4,9 +4,9 @@
 //
 // Per token row (position p) and channel c of q, k or v (u: the projection, rounded to the
 // activation type):
-//   conv    y_p = sum_j w[c, j] u_(p - taps + 1 + j)     (no weights: y = u); zeros
-//           before the sequence's start; earlier tokens of the sequence that are not in this step
-//           come from its state slot, which holds the last taps - 1 projected values
+//   conv    y[p] = sum over lags d < taps of w[c, taps - 1 - d] u[p - d]   (no weights: y = u);
+//           u is 0 ahead of token 0; tokens of earlier steps come from the sequence's state slot,
+//           which carries its taps - 1 newest projected values
 //   rotate  (q, k) the first rot_dims entries of every head turn by the position: pairs
 //           (i, i + rot_dims/2) when half, else (2i, 2i + 1); angle p * inv_freq[i]; cos, sin * amp
 //   norm    (q, k) every head divided by its root mean square, sqrt(mean + eps)

@@ -351,80 +351,81 @@ window_attn_kernel(const WinAttnArgs a) {
 
     // weights mixed across the heads need every head's final (max, sum): the keys are walked
     // twice, first for those, then for the weights
-    for (int pass = a.talk_post ? 0 : 1; pass < 2; ++pass)
-    for (int k0 = 0; k0 < nkeys; k0 += WA_KT) {
-      const int kk = k0 + lane;
-      const bool valid = kk < nkeys;
-      const int j = valid ? (kk < nsink ? kk : lo + kk - nsink) : pos;
-      const long slot = (long)bt[j / a.bs] * a.bs + j % a.bs;
-      __syncthreads();                                 // qs / mrun ready; last tile's reads over
-      if (wave == 0) vbase[lane] = (long)bt[j / a.bs] * vrow * a.bs + j % a.bs;
-      // (1) raw scores of this lane's key
-      for (int m = wave; m < M; m += 4) {
-        const int h = m / P, c = m - h * P;
-        const T* kp = kc + slot * krow + ((h / rep) * P + c) * D;
-        const float* qp = qs + m * D;
-        float s = 0.f;
-        for (int d = 0; d < D; ++d) s += qp[d] * ld_f32<T>(kp, d);
-        s *= a.mult[m];
-        if (a.slope) s -= a.slope[m] * (float)(pos - j);
-        if (a.cap > 0.f) s = a.cap * tanhf(s / a.cap);
-        if (a.talk_post && pass == 1)                  // the head's own final weight
-          s = valid ? expf(s - mrun[m]) / lrun[m] : 0.f;
-        sraw[m * WA_KT + lane] = s;
-      }
-      __syncthreads();
-      if (a.talk_post && pass == 1) {                  // mix the weights; nothing to rescale
+    for (int pass = a.talk_post ? 0 : 1; pass < 2; ++pass) {
+      for (int k0 = 0; k0 < nkeys; k0 += WA_KT) {
+        const int kk = k0 + lane;
+        const bool valid = kk < nkeys;
+        const int j = valid ? (kk < nsink ? kk : lo + kk - nsink) : pos;
+        const long slot = (long)bt[j / a.bs] * a.bs + j % a.bs;
+        __syncthreads();                                 // qs / mrun ready; last tile's reads over
+        if (wave == 0) vbase[lane] = (long)bt[j / a.bs] * vrow * a.bs + j % a.bs;
+        // (1) raw scores of this lane's key
         for (int m = wave; m < M; m += 4) {
-          float p = 0.f;
-          for (int g = 0; g < M; ++g) p += a.talk[m * M + g] * sraw[g * WA_KT + lane];
-          pw[m * WA_KT + lane] = p;
-          if (lane == 0) alpha[m] = 1.f;
+          const int h = m / P, c = m - h * P;
+          const T* kp = kc + slot * krow + ((h / rep) * P + c) * D;
+          const float* qp = qs + m * D;
+          float s = 0.f;
+          for (int d = 0; d < D; ++d) s += qp[d] * ld_f32<T>(kp, d);
+          s *= a.mult[m];
+          if (a.slope) s -= a.slope[m] * (float)(pos - j);
+          if (a.cap > 0.f) s = a.cap * tanhf(s / a.cap);
+          if (a.talk_post && pass == 1)                  // the head's own final weight
+            s = valid ? expf(s - mrun[m]) / lrun[m] : 0.f;
+          sraw[m * WA_KT + lane] = s;
         }
-      } else {
-      // (2) head mixing, mask, online softmax
-      for (int m = wave; m < M; m += 4) {
-        float s;
-        if (a.talk && !a.talk_post) {
-          s = 0.f;
-          for (int g = 0; g < M; ++g) s += a.talk[m * M + g] * sraw[g * WA_KT + lane];
+        __syncthreads();
+        if (a.talk_post && pass == 1) {                  // mix the weights; nothing to rescale
+          for (int m = wave; m < M; m += 4) {
+            float p = 0.f;
+            for (int g = 0; g < M; ++g) p += a.talk[m * M + g] * sraw[g * WA_KT + lane];
+            pw[m * WA_KT + lane] = p;
+            if (lane == 0) alpha[m] = 1.f;
+          }
         } else {
-          s = sraw[m * WA_KT + lane];
+          // (2) head mixing, mask, online softmax
+          for (int m = wave; m < M; m += 4) {
+            float s;
+            if (a.talk && !a.talk_post) {
+              s = 0.f;
+              for (int g = 0; g < M; ++g) s += a.talk[m * M + g] * sraw[g * WA_KT + lane];
+            } else {
+              s = sraw[m * WA_KT + lane];
+            }
+            if (a.wmode == 1) {                            // plain sigmoid weights: nothing to rescale
+              const float z = s + (a.bias ? a.bias[m] : 0.f);
+              pw[m * WA_KT + lane] = valid ? 1.0f / (1.0f + expf(-z)) : 0.f;
+              if (lane == 0) { alpha[m] = 1.f; lrun[m] = 1.f; }
+              continue;
+            }
+            if (!valid) s = -INFINITY;
+            const float mo = mrun[m];
+            const float mn = fmaxf(mo, wave_max(s));
+            const float p = valid ? expf(s - mn) : 0.f;
+            const float ps = wave_sum(p);
+            pw[m * WA_KT + lane] = p;
+            if (lane == 0) {
+              const float al = expf(mo - mn);              // exp(-inf) = 0 at the first tile
+              alpha[m] = al;
+              lrun[m] = lrun[m] * al + ps;
+              mrun[m] = mn;
+            }
+          }
         }
-        if (a.wmode == 1) {                            // plain sigmoid weights: nothing to rescale
-          const float z = s + (a.bias ? a.bias[m] : 0.f);
-          pw[m * WA_KT + lane] = valid ? 1.0f / (1.0f + expf(-z)) : 0.f;
-          if (lane == 0) { alpha[m] = 1.f; lrun[m] = 1.f; }
-          continue;
-        }
-        if (!valid) s = -INFINITY;
-        const float mo = mrun[m];
-        const float mn = fmaxf(mo, wave_max(s));
-        const float p = valid ? expf(s - mn) : 0.f;
-        const float ps = wave_sum(p);
-        pw[m * WA_KT + lane] = p;
-        if (lane == 0) {
-          const float al = expf(mo - mn);              // exp(-inf) = 0 at the first tile
-          alpha[m] = al;
-          lrun[m] = lrun[m] * al + ps;
-          mrun[m] = mn;
-        }
-      }
-      }
-      if (pass == 0) continue;                         // (uniform)
-      __syncthreads();
-      // (3) weighted values
-      const int nk = min(WA_KT, nkeys - k0);
-#pragma unroll
-      for (int i = 0; i < WA_ACC; ++i) {
-        const int idx = tid + i * 256;
-        if (idx < M * Dv) {
-          const int m = idx / Dv, d = idx - m * Dv;
-          const T* vp = vc + (long)(((m / P) / rep) * Dv + d) * a.bs;
-          const float* pm = pw + m * WA_KT;
-          float s = acc[i] * alpha[m];
-          for (int k = 0; k < nk; ++k) s += pm[k] * ld_f32<T>(vp, vbase[k]);
-          acc[i] = s;
+        if (pass == 0) continue;                         // (uniform)
+        __syncthreads();
+        // (3) weighted values
+        const int nk = min(WA_KT, nkeys - k0);
+  #pragma unroll
+        for (int i = 0; i < WA_ACC; ++i) {
+          const int idx = tid + i * 256;
+          if (idx < M * Dv) {
+            const int m = idx / Dv, d = idx - m * Dv;
+            const T* vp = vc + (long)(((m / P) / rep) * Dv + d) * a.bs;
+            const float* pm = pw + m * WA_KT;
+            float s = acc[i] * alpha[m];
+            for (int k = 0; k < nk; ++k) s += pm[k] * ld_f32<T>(vp, vbase[k]);
+            acc[i] = s;
+          }
         }
       }
     }

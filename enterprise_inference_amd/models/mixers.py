@@ -740,17 +740,18 @@ class MixAttentionMixer(_WindowMixerBase):
     """Grouped-query softmax attention over the part of a caller's fused projection that holds q,
     k and v (no biases); the caller owns the projection and the output product.  Options:
 
-    * ``taps`` > 0: y_t = sum_j w[c, j] u_(t - taps + 1 + j) on every channel c of q, k and v, zeros
-      before the sequence's start (weights ``q_conv`` / ``k_conv`` / ``v_conv`` [channels, taps]);
-      a state slot keeps each sequence's last taps - 1 projected values
+    * ``taps`` > 0: every projected channel u of q, k and v is filtered over time, y[t] = sum over
+      lags d < taps of w[taps - 1 - d] u[t - d], u being 0 ahead of token 0 (weights ``q_conv`` /
+      ``k_conv`` / ``v_conv`` [channels, taps], newest token last); a state slot carries the
+      taps - 1 newest projected values of each sequence
     * rotation of the first ``rot_dims`` entries of every q / k head (pairs (i, i + rot_dims/2));
       ``rot_scaling`` as in ops/rotary.py rotary_frequencies
     * ``qk_norm``: rotated queries and keys are divided by their root mean square per head
     * score = (q . k) * scale, then cap * tanh(score / cap) with ``softcap``; ``window`` 0 sees
       every earlier token
     * ``head_mix``: the softmax weights are mixed, w_h <- sum_g talk[h, g] w_g, before the values
-    * ``v_mix`` "first": the layer's values are the step's ValueCarry; "later": v <- (1 - vmix) v +
-      vmix * carry, and the mixed v is what is cached."""
+    * ``v_mix`` "first": the layer's values are the step's ValueCarry; "later": the cache receives
+      v + vmix * (carry - v)."""
 
     def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, scale: float, rot_dims: int,
                  rot_base: float, rot_scaling, eps: float, dtype, device, *, offsets: dict,

@@ -75,9 +75,9 @@ def rotary_frequencies(dims: int, base: float, scaling: Optional[dict] = None, d
     (YaRN) the pairs that turn fewer than ``slow`` times over ``original`` positions are slowed
     by ``factor``, those that turn more than ``fast`` times keep their frequency, the ones
     between are blended linearly in the pair index, and amp = 0.1 ln(factor) + 1.  With ``scaling``
-    = {factor, original, low, high} (Llama 3.1) the bands are set by wavelength, l = 2 pi / f: below
-    original/high f stays, above original/low it is divided by ``factor``, and between the two
-    blended with s = (original/l - low) / (high - low); amp = 1.  A ``scaling`` that gives only
+    = {factor, original, low, high} (Llama 3.1) the bands are set by the turns a pair makes over
+    ``original`` positions, t = original f / (2 pi): above ``high`` f stays, below ``low`` it is divided
+    by ``factor``, and in between the two are blended linearly in t; amp = 1.  A ``scaling`` that gives only
     ``factor`` is linear position interpolation: every f_i is divided by it.
     Evaluated in float64 and rounded once."""
     import math

@@ -147,7 +147,7 @@ def case_act_mul_embed(device, dtype):
     from enterprise_inference_amd.ops import activation as act
     from enterprise_inference_amd.ops.gemm import SplitK
     g = torch.Generator().manual_seed(3)
-    for n, pad, layers, T in ((5, 128, 3, 7), (24, 24, 2, 1), (130, 256, 2, 9), (128, 128, 1, 3)):
+    for n, pad, layers, T in ((5, 128, 3, 7), (28, 28, 2, 1), (130, 256, 2, 9), (128, 128, 1, 3)):
         table = torch.randn(31, layers * n, generator=g).to(dtype)
         ids = torch.randint(0, 31, (T,), generator=g).to(torch.int32)
         u = (torch.randn(T, pad, generator=g) * 2).to(dtype)
@@ -168,7 +168,7 @@ def case_act_mul_embed(device, dtype):
     assert torch.equal(act.softcap_(x.clone().to(device), 0.0).cpu(), x)
 
 
-def case_token_side(W=256, n=24, T=300, sublayers=2, nxt=True):
+def case_token_side(W=288, n=28, T=300, sublayers=2, nxt=True):
     """The whole layer end in one launch (bf16, prompt-sized): a last workgroup that is partly
     empty, one or two sublayers, gates as columns of a wider row, side widths below, at and above
     the padding unit, widths that do not fill the last wave's tiles, with and without a next norm."""

@@ -1,9 +1,9 @@
 """Plain float64 implementation of the Borosun design, written from its equations: loops over
 tokens, heads and keys, one function per mechanism, no code shared with the framework.
 
-A layer reads one RMS norm of the residual and adds both sublayers to it, each multiplied element
-by element by a sigmoid gate of the same normed input; a per-layer token embedding then joins
-through a gated low-width projection whose output is RMS-normed.  Mixers: ``attention`` (short
+A layer reads one RMS norm of the residual and adds both sublayers to it, each scaled by an
+element-wise sigmoid gate computed from the same normed input; a per-layer token embedding then
+joins through a gated low-width projection whose output is RMS-normed.  Mixers: ``attention`` (short
 causal convolutions on q, k and v, rotation with banded frequency scaling, softmax weights mixed
 across the heads, value mixing with the first such layer's values), ``attention_2`` (rotation,
 weightless RMS norm of q and k per head, soft-capped scores, sliding window, value mixing) and
@@ -77,7 +77,7 @@ def rotate(v, pos, rot):
 
 
 def short_conv(u, w):
-    """u: projected rows [T][C] of one sequence; w [C, taps]; zeros before the start."""
+    """u: projected rows [T][C] of one sequence; w [C, taps], newest token last."""
     taps = w.shape[1]
     out = []
     for t in range(len(u)):
