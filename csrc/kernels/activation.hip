@@ -89,27 +89,6 @@ EIA_API int eia_act(void* out, const void* x, long numel, int kind, hipStream_t 
   EIA_LAUNCH_CHECK();
 }
 
-// Squared ReLU, out = max(x, 0)^2, for bf16 or fp32 activations (ungated expert MLPs).
-template <typename T>
-__global__ void __launch_bounds__(256)
-relu2_kernel(T* __restrict__ out, const T* __restrict__ x, long n) {
-  for (long i = (long)blockIdx.x * 256 + threadIdx.x; i < n; i += (long)gridDim.x * 256) {
-    const float v = fmaxf(ld_f32<T>(x, i), 0.f);
-    st_f32<T>(out, i, v * v);
-  }
-}
-
-EIA_API int eia_relu2(void* out, const void* x, long numel, int is_bf16, hipStream_t st) {
-  if (numel < 0) return EIA_BAD_SHAPE;
-  if (numel == 0) return EIA_OK;
-  dim3 grid(grid_for((numel + 3) / 4)), block(256);
-  if (is_bf16)
-    hipLaunchKernelGGL(relu2_kernel<bf16_t>, grid, block, 0, st, (bf16_t*)out, (const bf16_t*)x, numel);
-  else
-    hipLaunchKernelGGL(relu2_kernel<float>, grid, block, 0, st, (float*)out, (const float*)x, numel);
-  EIA_LAUNCH_CHECK();
-}
-
 // Gated activation straight from the fp32 split-K partials [sk, T, 2F] of a [gate; up] GEMM:
 // out[T, F] = act(sum_z gate_z) * (sum_z up_z), four columns per thread.
 template <int KIND>
@@ -205,6 +184,59 @@ xielu_kernel(const T* __restrict__ x, long ldx, const float* __restrict__ part, 
   if (idx >= (long)rows * F) return;
   const int row = idx / F, col = idx % F;
   st_f32<T>(out + (long)row * ldo, col, xielu_f(ld_f32<T>(x + (long)row * ldx, col), ap, aq));
+}
+
+// Squared ReLU, out = max(x, 0)^2, of rows [rows, F] (type T, row stride ldx) or of the fp32 split-K
+// partials [sk, rows, F] of the GEMM that produced them (summed here, F % 4 == 0).  V: elements per
+// thread (4: F, ldx and the pointers allow 8- / 16-byte accesses).
+template <typename T, int V>
+__global__ void __launch_bounds__(256)
+relu2_kernel(const T* __restrict__ x, long ldx, const float* __restrict__ part, int sk,
+             T* __restrict__ out, long ldo, int rows, int F) {
+  const long idx = ((long)blockIdx.x * 256 + threadIdx.x) * V;
+  if (idx >= (long)rows * F) return;
+  const int row = idx / F, col = idx % F;
+  if constexpr (V == 4) {
+    f32x4 v;
+    if (part) {
+      const float* p = part + idx;
+      v = *reinterpret_cast<const f32x4*>(p);
+#pragma unroll 4
+      for (int z = 1; z < sk; ++z) v += *reinterpret_cast<const f32x4*>(p + z * ((long)rows * F));
+    } else {
+      v = act_ld4<T>(x + row * ldx + col);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const float r = fmaxf(v[i], 0.f);
+      v[i] = r * r;
+    }
+    act_st4<T>(out + row * ldo + col, v);
+  } else {
+    const float r = fmaxf(ld_f32<T>(x + row * ldx, col), 0.f);
+    st_f32<T>(out + row * ldo, col, r * r);
+  }
+}
+
+EIA_API int eia_relu2(const void* x, long ldx, const float* part, int sk, void* out, long ldo,
+                      int rows, int F, int is_bf16, hipStream_t st) {
+  if (rows < 0 || F < 1 || !out || (x == nullptr) == (part == nullptr) ||
+      (part && (sk < 1 || F % 4 || ldo % 4)))
+    return EIA_BAD_SHAPE;
+  if (rows == 0) return EIA_OK;
+  const int esz = is_bf16 ? 2 : 4;
+  const bool vec = part || (F % 4 == 0 && ldx % 4 == 0 && ldo % 4 == 0 &&
+                            ((reinterpret_cast<uintptr_t>(x) | reinterpret_cast<uintptr_t>(out)) %
+                             (4 * esz)) == 0);
+  const long n = (long)rows * F / (vec ? 4 : 1);
+  const dim3 grid((unsigned)((n + 255) / 256)), block(256);
+#define RELU2(TT, VV)                                                                          \
+  hipLaunchKernelGGL((relu2_kernel<TT, VV>), grid, block, 0, st, (const TT*)x, ldx, part, sk, \
+                     (TT*)out, ldo, rows, F)
+  if (is_bf16) { if (vec) RELU2(bf16_t, 4); else RELU2(bf16_t, 1); }
+  else { if (vec) RELU2(float, 4); else RELU2(float, 1); }
+#undef RELU2
+  EIA_LAUNCH_CHECK();
 }
 
 EIA_API int eia_xielu(const void* x, long ldx, const float* part, int sk, long ldp, const void* pq,

@@ -21,7 +21,8 @@
 //            key or a value, not scaled, counted once.  The running (max, sum) of a row simply
 //            starts at (sink, 1) instead of (-inf, 0); with key partitions, in partition 0.
 //
-// Epilogue 0: out[h] = a_h * sigmoid(gate[h]) * post   (gate == nullptr: no gate; P must be 1)
+// Epilogue 0: out[h] = a_h * sigmoid(gate[h]) * post   (gate == nullptr: no gate; P must be 1);
+//             a gate value per value column, or with gate_heads one per head
 // Epilogue 1: o = a_{2h} - lam * a_{2h+1};  out[h] = o / sqrt(mean(o^2) + eps) * post   (P == 2;
 //             lam is read from device memory, so a captured launch follows a weight reload)
 //
@@ -263,6 +264,7 @@ struct WinAttnArgs {
   const float* sink;                // [M] or null (wmode 0)
   float cap;                        // > 0: scores soft-capped, cap * tanh(s / cap)
   int talk_post;                    // talk mixes the softmax weights, not the scores (scalar form)
+  int gate_heads;                   // gate [rows, H]: one value per head
 };
 
 // The visible keys of a 16-query tile as absolute 32-key blocks: the blocks of the kept first
@@ -436,7 +438,8 @@ window_attn_kernel(const WinAttnArgs a) {
         const int idx = tid + i * 256;
         if (idx < M * Dv) {
           float v = (a.talk_post ? acc[i] : acc[i] / lrun[idx / Dv]) * a.post;
-          if (gate) v *= 1.0f / (1.0f + expf(-ld_f32<T>(gate + row * a.ldg, idx)));
+          if (gate)
+            v *= 1.0f / (1.0f + expf(-ld_f32<T>(gate + row * a.ldg, a.gate_heads ? idx / Dv : idx)));
           st_f32<T>(out + row * a.ldo, idx, v);
         }
       }
@@ -477,7 +480,7 @@ EIA_API int eia_window_attn(const void* q, long ldq, const void* kc, const void*
                             int H, int G, int P, int D, int Dv, int bs, int window, int keep,
                             int qb, int epilogue, const float* lam, float eps, float post,
                             int wmode, const float* bias, const float* sink, float cap,
-                            int talk_post, int is_bf16, hipStream_t st) {
+                            int talk_post, int gate_heads, int is_bf16, hipStream_t st) {
   if (n_items < 0 || H < 1 || G < 1 || H % G || (P != 1 && P != 2) || D < 1 || Dv < 1 || bs < 1 ||
       keep < 0 || qb < 1 || !q || !kc || !vc || !bt || !positions || !mult || !out)
     return EIA_BAD_SHAPE;
@@ -492,7 +495,7 @@ EIA_API int eia_window_attn(const void* q, long ldq, const void* kc, const void*
   if (n_items == 0) return EIA_OK;
   WinAttnArgs a{q, ldq, kc, vc, bt, ldbt, positions, cu, work, lens, mult, slope, talk, gate, ldg,
                 out, ldo, H, G, P, D, Dv, bs, window, keep, qb, epilogue, lam, eps, post, 1, 2,
-                nullptr, nullptr, wmode, bias, sink, cap, talk_post};
+                nullptr, nullptr, wmode, bias, sink, cap, talk_post, gate_heads};
   if (is_bf16)
     hipLaunchKernelGGL((window_attn_kernel<bf16_t>), dim3(n_items), dim3(256), lds, st, a);
   else
@@ -838,7 +841,9 @@ window_attn_mfma_kernel(const WinAttnArgs a) {
     const bf16_t* gate = (const bf16_t*)a.gate;
 #pragma unroll
     for (int m = 0; m < MW; ++m) {
-      const float inv = a.post / lrun[m];
+      float inv = a.post / lrun[m];
+      if (gate && a.gate_heads)
+        inv *= 1.0f / (1.0f + __expf(-bf2f(gate[row * a.ldg + h0 + m])));
 #pragma unroll
       for (int t = 0; t < NDV; ++t) {
         if (t < ndv) {
@@ -847,7 +852,8 @@ window_attn_mfma_kernel(const WinAttnArgs a) {
 #pragma unroll
           for (int i = 0; i < 4; ++i) {
             float v = acc[m][t][i] * inv;
-            if (gate) v *= 1.0f / (1.0f + __expf(-bf2f(gate[row * a.ldg + col + i])));
+            if (gate && !a.gate_heads)
+              v *= 1.0f / (1.0f + __expf(-bf2f(gate[row * a.ldg + col + i])));
             o[i] = f2bf(v);
           }
           *reinterpret_cast<bf16x4*>(out + row * a.ldo + col) = o;
@@ -920,7 +926,11 @@ window_attn_merge_kernel(const WinAttnArgs a) {
     const bf16_t* gate = (const bf16_t*)a.gate;
     r0 = o[0][0] * a.post;
     r1 = o[0][1] * a.post;
-    if (gate) {
+    if (gate && a.gate_heads) {
+      const float gs = 1.0f / (1.0f + __expf(-bf2f(gate[row * a.ldg + h])));
+      r0 *= gs;
+      r1 *= gs;
+    } else if (gate) {
       if (lane < Dv) r0 *= 1.0f / (1.0f + __expf(-bf2f(gate[row * a.ldg + h * Dv + lane])));
       if (lane + 64 < Dv) r1 *= 1.0f / (1.0f + __expf(-bf2f(gate[row * a.ldg + h * Dv + lane + 64])));
     }
@@ -961,7 +971,7 @@ EIA_API int eia_window_attn_mfma(const void* q, long ldq, const void* kc, const 
                                  int window, int keep, int epilogue, const float* lam, float eps,
                                  float post, int wmode, const float* bias, int nparts,
                                  float* part_acc, float* part_ml, const float* sink, float cap,
-                                 hipStream_t st) {
+                                 int gate_heads, hipStream_t st) {
   if (n_items < 0 || H < 1 || G < 1 || H % G || (P != 1 && P != 2) || bs < 1 || keep < 0 || !q ||
       !kc || !vc || !bt || !positions || !mult || !out)
     return EIA_BAD_SHAPE;
@@ -977,7 +987,7 @@ EIA_API int eia_window_attn_mfma(const void* q, long ldq, const void* kc, const 
   if (n_items == 0) return EIA_OK;
   WinAttnArgs a{q, ldq, kc, vc, bt, ldbt, positions, cu, work, lens, mult, slope, talk, gate, ldg,
                 out, ldo, H, G, P, D, Dv, bs, window, keep, 16, epilogue, lam, eps, post, nparts,
-                2, part_acc, part_ml, wmode, bias, sink, cap, 0};
+                2, part_acc, part_ml, wmode, bias, sink, cap, 0, gate_heads};
   // raw-score buffers of the head-mixing form: two (one barrier per block) while they fit 48 KiB
   if (talk) a.raw_bufs = (size_t)2 * H * P * 128 * sizeof(f32x4) > 48 * 1024 ? 1 : 2;
   // sigmoid weights: a wave takes two heads of one kv head where the grouping allows it, so the

@@ -83,16 +83,23 @@ _SIGNATURES = {
                                 P, P, F, I, P, S],
     "eia_hyper_step": [P, I, I, P, L, P, I, P, P, P, F, P, P, F, P, L, F, I, I, S],
     "eia_bigram_embed": [IP, P, F, P, I, L, L, IP, IP, IP, I, IP, P, I, I, I, I, I, S],
-    "eia_relu2": [P, P, L, I, S],
+    "eia_relu2": [P, L, P, I, P, L, I, I, I, S],
+    "eia_delta_prep": [P, L, P, I, L, I, I, I, I, I, I, I, I, I, I, P, P, P, I, P, P, P, F, IP, IP,
+                       IP, IP, I, I, P, P, P, I, I, P, P, P, L, I, I, P, I, I, I, I, I, I, I, P, I,
+                       I, F, IP, P, L, P, P, I, I, S],
+    "eia_delta_scan": [P, P, P, P, P, I, I, I, I, I, I, P, L, P, F, F, P, IP, IP, IP, IP, P, L, I, I,
+                       S],
+    "eia_delta_scan_chunked": [P, P, P, P, P, I, I, I, I, I, I, P, L, P, F, F, P, IP, IP, P, L, I, IP,
+                               IP, I, P, P, P, P, P, I, S],
     "eia_moe_combine_postnorm": [P, L, P, P, I, P, L, P, F, P, P, L, I, I, I, S],
     "eia_gnorm": [P, L, P, I, P, P, P, P, P, P, L, F, I, I, I, I, S],
     "eia_splitk_act_and_mul": [P, I, I, I, P, L, I, S],
     "eia_qk_norm_cache": [P, L, P, I, P, I, I, I, I, I, I, I, I, I, P, P, P, L, P, P, P, L, IP, I, F,
                           I, I, S],
     "eia_window_attn": [P, L, P, P, IP, I, IP, IP, IP, IP, I, P, P, P, P, L, P, L, I, I, I, I, I,
-                        I, I, I, I, I, P, F, F, I, P, P, F, I, I, S],
+                        I, I, I, I, I, P, F, F, I, P, P, F, I, I, I, S],
     "eia_window_attn_mfma": [P, L, P, P, IP, I, IP, IP, IP, IP, I, P, P, P, P, L, P, L, I, I, I, I,
-                             I, I, I, I, I, P, F, F, I, P, I, P, P, P, F, S],
+                             I, I, I, I, I, P, F, F, I, P, I, P, P, P, F, I, S],
     "eia_head_mix_attn": [P, L, P, P, IP, I, IP, IP, IP, IP, I, I, P, P, P, L, I, I, I, I, I, I, F,
                           F, I, P, P, S],
     "eia_head_mix_attn_ok": [I, I, I, I, I],

@@ -139,13 +139,15 @@ class ModelConfig:
     def from_layer_list(cls, d: Dict[str, Any], name: str = "",
                         tensor_shapes: Optional[Dict[str, Any]] = None) -> "ModelConfig":
         """Designs whose config.json names the architecture in one string and lists the layers
-        one by one (Sekolorn, Vedadra, Gapidra, Daburax, Borosun): keys ``architecture``,
-        ``vocab``, ``width``, ``norm.eps`` and ``layers`` (kept whole in ``extra["layers"]``);
+        one by one (Sekolorn, Vedadra, Gapidra, Daburax, Borosun, Vugelix): keys
+        ``architecture``, ``vocab``, ``width``, ``norm.eps`` and ``layers`` (kept whole in
+        ``extra["layers"]``);
         ``norm``, ``embedding`` ({scale, bigram}) and an optional ``loop`` ({start, stop, times}: a
         run of layers repeated with the same weights) are kept whole too, as are
         ``residual_mult`` (a factor on every sublayer output), ``streams`` (residual copies joined
-        by hyper-connections), ``token_side`` ({dim}: a per-layer token embedding) and
-        ``logit_softcap``.  Sizes the file leaves to the checkpoint (the rank of a wkv or gla
+        by hyper-connections), ``token_side`` ({dim}: a per-layer token embedding),
+        ``logit_softcap`` and ``logit_scale``.  A layer may run another layer's tensors
+        (``weights_of``).  Sizes the file leaves to the checkpoint (the rank of a wkv or gla
         layer's decay branch) come from ``tensor_shapes`` when given."""
         import copy
         layers = copy.deepcopy(d["layers"])
@@ -170,7 +172,8 @@ class ModelConfig:
                                      "residual_mult": d.get("residual_mult"),
                                      "streams": d.get("streams"),
                                      "token_side": dict(d.get("token_side") or {}),
-                                     "logit_softcap": d.get("logit_softcap")})
+                                     "logit_softcap": d.get("logit_softcap"),
+                                     "logit_scale": d.get("logit_scale")})
 
     @classmethod
     def from_hf_dict(cls, d: Dict[str, Any], name: str = "") -> "ModelConfig":

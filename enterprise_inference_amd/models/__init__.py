@@ -22,6 +22,7 @@ _REGISTRY: Dict[str, str] = {
     "Gapidra": "gapidra:GapidraForCausalLM",
     "Daburax": "daburax:DaburaxForCausalLM",
     "Borosun": "borosun:BorosunForCausalLM",
+    "Vugelix": "vugelix:VugelixForCausalLM",
     "BertModel": "bert:BertEmbeddingModel",
     "XLMRobertaModel": "bert:BertEmbeddingModel",
     "XLMRobertaForSequenceClassification": "bert:CrossEncoderModel",

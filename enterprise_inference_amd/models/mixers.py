@@ -20,9 +20,10 @@ returns the mixer output in the activation dtype.
 * ``SigmoidWindowAttentionMixer`` -- grouped-query sliding-window attention whose weights are
   ``sigmoid(score + bias_h)``, not normalised over the keys; queries and keys are RMS-normed as
   whole projections and then rotated.
-* ``SinkAttentionMixer`` -- grouped-query causal softmax attention with projection biases, a
-  partial rotation with optional position interpolation and a learned per-head sink in the
-  softmax denominator (optionally windowed).
+* ``SinkAttentionMixer`` -- grouped-query causal softmax attention with a sink in the softmax
+  denominator (learned per head, or one unit) and a partial rotation with optional position
+  interpolation; optional projection biases, window, soft cap on the scores and sigmoid gate per
+  head.
 * ``MixAttentionMixer`` -- grouped-query softmax attention whose options are a short causal
   convolution over time on q, k and v, a weightless RMS norm of the rotated queries and keys, a
   soft cap on the scores, a sliding window, mixing of the softmax weights across the heads, and
@@ -36,9 +37,12 @@ returns the mixer output in the activation dtype.
 * ``GatedLinearMixer`` -- gated linear attention: a matrix state per head whose rows decay per key
   channel by a data-dependent low-rank branch, head RMS norm with a shared weight, SiLU gate.
   All three run ops/linear_scan.py.
-* ``ParallelMixer`` -- an attention mixer and a recurrent mixer side by side on the same input:
-  one fused input projection, one output projection over the concatenated heads, the two
-  outputs added with fixed factors.
+* ``GatedDeltaMixer`` -- gated delta rule: short convolutions on q, k and v, unit-length queries and
+  keys, a decay and a step size per head and token, head RMS norm with a shared weight, SiLU gate
+  (ops/delta_scan.py).
+* ``ParallelMixer`` / ``WindowDeltaMixer`` -- an attention mixer and a recurrent mixer side by side
+  on the same input: one fused input projection, one output projection over the concatenated heads,
+  the two outputs added with fixed factors.
 """
 
 from __future__ import annotations
@@ -47,6 +51,7 @@ import torch
 import torch.nn as nn
 
 from ..ops import activation as act_ops
+from ..ops import delta_scan as delta_ops
 from ..ops import gemm
 from ..ops import latent_attention as lat_ops
 from ..ops import linear_scan as scan_ops
@@ -496,53 +501,73 @@ class FusedProjection(nn.Module):
 
 
 class SinkAttentionMixer(_WindowMixerBase):
-    """Grouped-query causal softmax attention: q, k and v carry biases; the first ``rot_dims``
-    entries of every query / key head turn by the position (pairs (2i, 2i+1), or (i, i +
+    """Grouped-query causal softmax attention: q, k and v carry biases (``bias``); the first
+    ``rot_dims`` entries of every query / key head turn by the position (pairs (2i, 2i+1), or (i, i +
     rot_dims/2) with ``rot_half``; ``rot_scaling`` as in ops/rotary.py rotary_frequencies, a
-    lone ``factor`` divides every frequency); score = (q . k) * scale; the softmax denominator
-    of head h also holds exp(sink_h), a learned term without key or value; ``window`` 0 sees
-    every earlier token.  The concatenated heads are multiplied by ``out_scale``.
-    ``proj`` / ``prefix``: the q, k, v parts live in a caller's FusedProjection under
+    lone ``factor`` divides every frequency); score = (q . k) * scale, soft-capped with ``softcap``
+    > 0, cap * tanh(score / cap); the softmax denominator of head h also holds exp(sink_h), a term
+    without key or value that is learned (``sink`` "learned") or exp(0) ("unit"); ``window`` 0 sees
+    every earlier token.  ``head_gate``: head h's output is multiplied by sigmoid(W_g x)_h (rows
+    ``g`` of the projection).  The concatenated heads are multiplied by ``out_scale``.
+    ``proj`` / ``prefix``: the q, k, v (g) parts live in a caller's FusedProjection under
     ``prefix + "q"`` ...; the caller then also owns the output projection, and ``attend`` writes
     the heads into the caller's buffer."""
 
-    PARTS = ("q", "k", "v")
-
     @staticmethod
-    def parts(heads, kv_heads, dim, vdim):
-        return [("q", heads * dim), ("k", kv_heads * dim), ("v", kv_heads * vdim)]
+    def parts(heads, kv_heads, dim, vdim, head_gate=False):
+        out = [("q", heads * dim), ("k", kv_heads * dim), ("v", kv_heads * vdim)]
+        return out + [("g", heads)] if head_gate else out
 
     def __init__(self, width: int, heads: int, kv_heads: int, dim: int, vdim: int, scale: float,
                  rot_dims: int, rot_base: float, rot_scaling, eps: float, dtype, device,
                  window: int = 0, rot_half: bool = False, out_scale: float = 1.0,
-                 proj: "FusedProjection" = None, prefix: str = ""):
+                 proj: "FusedProjection" = None, prefix: str = "", *, bias: bool = True,
+                 sink: str = "learned", softcap: float = 0.0, head_gate: bool = False):
         super().__init__()
         if rot_dims > dim or rot_dims % 2:
             raise ValueError("rot.dims must be even and at most dim")
+        if sink not in ("learned", "unit"):
+            raise ValueError(f"attention sink {sink!r}")
         own = proj is None
+        parts = self.parts(heads, kv_heads, dim, vdim, head_gate)
         self._setup(width, heads, kv_heads, dim, vdim, scale, window, 0, eps,
-                    self.parts(heads, kv_heads, dim, vdim) if own else [], own, dtype, device,
-                    norms=False, own_out=own)
+                    parts if own else [], own and bias, dtype, device, norms=False, own_out=own)
         if not own:
             self.proj = self.proj_bias = None
-            self.offsets = {n: proj.offsets[prefix + n] for n in self.PARTS}
-        self.rot_dims, self.rot_half = int(rot_dims), rot_half
-        self.inv_freq, self.rot_amp = rot_ops.rotary_frequencies(rot_dims, rot_base, rot_scaling,
-                                                                 device)
-        self.sink = _plain((heads,), dtype, device)
+            self.offsets = {n: proj.offsets[prefix + n] for n, _ in parts}
+        inv_freq, amp = rot_ops.rotary_frequencies(rot_dims, rot_base, rot_scaling, device)
+        # rotation and cache write, alone or inside another mixer's prep launch
+        self.prep = win_ops.PrepSpec(heads, kv_heads, dim, vdim, inv_freq, int(rot_dims), rot_half,
+                                     amp)
+        self.sink = _plain((heads,), dtype, device) if sink == "learned" else None
         self.spec.sink = torch.zeros(heads, dtype=torch.float32, device=device)
         self.spec.post = float(out_scale)
+        self.spec.cap = float(softcap)
+        self.head_gate = self.spec.gate_heads = bool(head_gate)
 
     def refresh(self) -> None:
-        self.spec.sink.copy_(self.sink.float())
+        if self.sink is not None:
+            self.spec.sink.copy_(self.sink.float())
+
+    def attn_prep(self, cache: PagedKVRows) -> delta_ops.AttnPrep:
+        g = self.offsets["g"] if self.head_gate else (0, 0)
+        return delta_ops.AttnPrep(self.offsets["q"][0], self.offsets["k"][0], self.offsets["v"][0],
+                                  self.prep, cache.k, cache.v, *g)
+
+    def attend_prepared(self, q, gate, md: AttentionMetadata, cache: PagedKVRows, out=None):
+        return win_ops.window_attention(q, cache.k, cache.v, md, self.spec, gate, out=out)
 
     def attend(self, fused, md: AttentionMetadata, cache: PagedKVRows, out=None):
+        if self.head_gate and isinstance(fused, gemm.SplitK):
+            fused = fused.materialize()            # (the gate columns are read by the attention)
+        p = self.prep
         q = win_ops.qk_rope_cache(fused, self.offsets["q"][0], self.offsets["k"][0],
                                   self.offsets["v"][0], self.heads, self.kv_heads, self.dim,
-                                  self.kv_heads * self.vdim, None, None, self.inv_freq,
-                                  self.rot_dims, self.rot_half, self.rot_amp, md.positions,
-                                  cache.k, cache.v, md.slot_mapping, self.eps)
-        return win_ops.window_attention(q, cache.k, cache.v, md, self.spec, None, out=out)
+                                  self.kv_heads * self.vdim, None, None, p.inv_freq, p.rot_dims,
+                                  p.rot_half, p.rot_amp, md.positions, cache.k, cache.v,
+                                  md.slot_mapping, self.eps)
+        gate = gemm.columns(fused, *self.offsets["g"]) if self.head_gate else None
+        return self.attend_prepared(q, gate, md, cache, out)
 
     def forward(self, xb: torch.Tensor, md: AttentionMetadata, cache: PagedKVRows):
         fused = gemm.linear(xb, self.proj, self.proj_bias, defer_reduce=True)
@@ -665,11 +690,108 @@ class MatrixMemoryMixer(_ScanMixerBase):
         return self._scan(fused, md, state, self.norm, out)
 
 
-class ParallelMixer(nn.Module):
-    """Two mixers side by side on the same input, ``left_scale * left(x) + right_scale *
-    right(x)``: ``left`` a SinkAttentionMixer on paged K / V rows, ``right`` a MatrixMemoryMixer on
-    state slots.  Both read ONE fused input projection and write their (scaled) heads into one
-    row, so one output projection over the concatenated heads adds the two in fp32."""
+class GatedDeltaMixer(nn.Module):
+    """Gated delta rule over the part of a caller's fused projection that holds q, k [kv_heads, dim],
+    v, g [heads, vdim], b and a [heads] (no biases); the caller owns the projection and the output
+    product.  q, k and v pass a short causal convolution over time (``q_conv`` / ``k_conv`` /
+    ``v_conv`` [channels, taps], newest token last) and silu; q and k become unit vectors per head, q
+    times dim^(-1/2); per head a decay exp(-exp(A_log) softplus(a + dt_bias)), a step size
+    sigmoid(b), and the recurrence of ops/delta_scan.py; every head's output is divided by its root
+    mean square and multiplied by ``norm`` [vdim], silu(W_g x) and ``out_scale``."""
+
+    PARTS = ("q", "k", "v", "g", "b", "a")
+
+    @staticmethod
+    def parts(heads, kv_heads, dim, vdim):
+        return [("q", kv_heads * dim), ("k", kv_heads * dim), ("v", heads * vdim),
+                ("g", heads * vdim), ("b", heads), ("a", heads)]
+
+    def __init__(self, heads: int, kv_heads: int, dim: int, vdim: int, taps: int, eps: float, dtype,
+                 device, *, proj: "FusedProjection", prefix: str = "", out_scale: float = 1.0):
+        super().__init__()
+        if pstate.tp_size() != 1:
+            raise NotImplementedError("recurrent mixers run on one rank (no head sharding yet)")
+        if heads % kv_heads:
+            raise ValueError("heads must be a multiple of kv_heads")
+        if not 1 <= taps <= win_ops.PREP_MAX_TAPS:
+            raise ValueError(f"short convolution: 1 to {win_ops.PREP_MAX_TAPS} taps")
+        self.offsets = {n: proj.offsets[prefix + n][0] for n in self.PARTS}
+        self.dtype = dtype
+        self.q_conv = _plain((kv_heads * dim, taps), dtype, device)
+        self.k_conv = _plain((kv_heads * dim, taps), dtype, device)
+        self.v_conv = _plain((heads * vdim, taps), dtype, device)
+        self.A_log = _plain((heads,), dtype, device)
+        self.dt_bias = _plain((heads,), dtype, device)
+        self.norm = _plain((vdim,), dtype, device)
+        # fp32 constants of the launches, refreshed IN PLACE after a weight load (captured decode
+        # graphs hold their addresses)
+        f32 = lambda: torch.zeros(heads, dtype=torch.float32, device=device)
+        self.spec = delta_ops.DeltaSpec(heads, kv_heads, dim, vdim, taps, self.q_conv, self.k_conv,
+                                        self.v_conv, f32(), f32(), float(dim) ** -0.5,
+                                        float(out_scale), float(eps))
+
+    def refresh(self) -> None:
+        self.spec.exp_a.copy_(torch.exp(self.A_log.float()))
+        self.spec.dt_bias.copy_(self.dt_bias.float())
+
+    def state_bytes(self, elem: int) -> int:
+        return delta_ops.DeltaState.slot_bytes(self.spec, elem)
+
+    def allocate_state(self, num_slots: int, dtype, device) -> delta_ops.DeltaState:
+        return delta_ops.DeltaState.allocate(num_slots, self.spec, dtype, device)
+
+    def prepare(self, fused, md: AttentionMetadata, state, attn=None) -> delta_ops.DeltaRows:
+        """``attn``: an attention mixer's share of the same rows, prepared by the same launch."""
+        return delta_ops.delta_prep(fused, self.offsets, self.spec, state, md, attn)
+
+    def attend(self, rows: delta_ops.DeltaRows, md: AttentionMetadata, state, out=None):
+        plan = delta_ops.prefill_plan(md, rows.q.device) if rows.q.is_cuda else None
+        return delta_ops.delta_scan(rows, self.spec, state, md, self.norm, out, plan)
+
+
+class _SideBySide(nn.Module):
+    """Two mixers on the same input, ``left_scale * left(x) + right_scale * right(x)``: both read ONE
+    fused input projection and write their (scaled) heads into one row, so one output projection over
+    the concatenated heads adds the two in fp32."""
+
+    def _setup_out(self, width: int, left_cols: int, right_cols: int, dtype, device) -> None:
+        self.lw, self.rw = left_cols, right_cols
+        self.lw_pad = -(-self.lw // 8) * 8           # the right heads start 16-byte aligned
+        self.row = -(-(self.lw_pad + self.rw) // 8) * 8     # ... and so does every row
+        # output projection over [left heads | pad | right heads | pad]; the checkpoint's two
+        # output matrices load into its column ranges (pad columns stay zero)
+        self.o = _param((width, self.row), dtype, device)
+        self.o.data.zero_()
+        self.o.weight_loader = self._load_o
+
+    def _load_o(self, param, loaded, shard_id=None):
+        off, n = (0, self.lw) if shard_id == "left" else (self.lw_pad, self.rw)
+        if loaded.shape != (param.shape[0], n):
+            raise ValueError(f"parallel mixer {shard_id}.o: shape {tuple(loaded.shape)}")
+        param.data[:, off:off + n].copy_(loaded)
+
+    def zero_pads(self) -> None:
+        """Pad columns of the output matrix back to zero (after a random fill of the whole)."""
+        self.o.data[:, self.lw:self.lw_pad].zero_()
+        self.o.data[:, self.lw_pad + self.rw:].zero_()
+
+    def refresh(self) -> None:
+        self.left.refresh()
+        self.right.refresh()
+
+    def _heads(self, xb: torch.Tensor):
+        """(the shared row [T, row], its left columns, its right columns)."""
+        heads = torch.empty(xb.shape[0], self.row, dtype=xb.dtype, device=xb.device)
+        if self.lw_pad != self.lw:
+            heads[:, self.lw:self.lw_pad].zero_()
+        if self.row != self.lw_pad + self.rw:
+            heads[:, self.lw_pad + self.rw:].zero_()
+        return heads, heads[:, :self.lw], heads[:, self.lw_pad:self.lw_pad + self.rw]
+
+
+class ParallelMixer(_SideBySide):
+    """``left`` a SinkAttentionMixer (biases, learned sinks) on paged K / V rows, ``right`` a
+    MatrixMemoryMixer on state slots."""
 
     def __init__(self, width: int, left: dict, right: dict, left_scale: float, right_scale: float,
                  eps: float, dtype, device):
@@ -690,38 +812,57 @@ class ParallelMixer(nn.Module):
         self.right = MatrixMemoryMixer(width, right["heads"], right["dim"], right["vdim"],
                                        right["gate_cap"], eps, dtype, device,
                                        out_scale=right_scale, proj=self.proj, prefix="right.")
-        self.lw = left["heads"] * left["vdim"]
-        self.rw = right["heads"] * right["vdim"]
-        self.lw_pad = -(-self.lw // 8) * 8           # the right heads start 16-byte aligned
-        self.row = -(-(self.lw_pad + self.rw) // 8) * 8     # ... and so does every row
-        # output projection over [left heads | pad | right heads | pad]; the checkpoint's two
-        # output matrices load into its column ranges (pad columns stay zero)
-        self.o = _param((width, self.row), dtype, device)
-        self.o.data.zero_()
-        self.o.weight_loader = self._load_o
-
-    def _load_o(self, param, loaded, shard_id=None):
-        off, n = (0, self.lw) if shard_id == "left" else (self.lw_pad, self.rw)
-        if loaded.shape != (param.shape[0], n):
-            raise ValueError(f"parallel mixer {shard_id}.o: shape {tuple(loaded.shape)}")
-        param.data[:, off:off + n].copy_(loaded)
-
-    def refresh(self) -> None:
-        self.left.refresh()
-        self.right.refresh()
+        self._setup_out(width, left["heads"] * left["vdim"], right["heads"] * right["vdim"], dtype,
+                        device)
 
     def forward(self, xb: torch.Tensor, md: AttentionMetadata, cache):
         """cache: (PagedKVRows of the left mixer, ScanState of the right one)."""
         kv, state = cache
         fused = self.proj(xb)
-        T = xb.shape[0]
-        heads = torch.empty(T, self.row, dtype=xb.dtype, device=xb.device)
-        if self.lw_pad != self.lw:
-            heads[:, self.lw:self.lw_pad].zero_()
-        if self.row != self.lw_pad + self.rw:
-            heads[:, self.lw_pad + self.rw:].zero_()
-        self.left.attend(fused, md, kv, out=heads[:, :self.lw])
-        self.right.attend(fused, md, state, out=heads[:, self.lw_pad:self.lw_pad + self.rw])
+        heads, lo, ro = self._heads(xb)
+        self.left.attend(fused, md, kv, out=lo)
+        self.right.attend(fused, md, state, out=ro)
+        # may return gemm.SplitK: the layer's boundary step reduces it
+        return gemm.linear(heads, self.o, defer_reduce=True)
+
+
+class WindowDeltaMixer(_SideBySide):
+    """``left`` a SinkAttentionMixer (no biases, a unit sink, half-split rotation pairs, sliding
+    window, soft-capped scores, a sigmoid gate per head) on paged K / V rows, ``right`` a
+    GatedDeltaMixer on state slots.  One launch prepares both sides from the projection rows
+    (decode-sized batches: straight from the projection GEMM's split-K partials)."""
+
+    def __init__(self, width: int, left: dict, right: dict, left_scale: float, right_scale: float,
+                 eps: float, dtype, device):
+        super().__init__()
+        lp = SinkAttentionMixer.parts(left["heads"], left["kv_heads"], left["dim"], left["vdim"],
+                                      head_gate=True)
+        rp = GatedDeltaMixer.parts(right["heads"], right["kv_heads"], right["dim"], right["vdim"])
+        self.proj = FusedProjection(
+            width, [("left." + n, r) for n, r in lp] + [("right." + n, r) for n, r in rp], dtype,
+            device)
+        rot = left.get("rot") or {}
+        self.left = SinkAttentionMixer(
+            width, left["heads"], left["kv_heads"], left["dim"], left["vdim"], left["scale"],
+            int(rot.get("dims", left["dim"] if rot else 0)), float(rot.get("base", 10000.0)),
+            rot.get("scaling"), eps, dtype, device,
+            window=int((left.get("mask") or {}).get("size", 0)), rot_half=True,
+            out_scale=left_scale, proj=self.proj, prefix="left.", bias=False, sink="unit",
+            softcap=float(left.get("softcap") or 0.0), head_gate=True)
+        self.right = GatedDeltaMixer(right["heads"], right["kv_heads"], right["dim"], right["vdim"],
+                                     right["conv"], eps, dtype, device, proj=self.proj,
+                                     prefix="right.", out_scale=right_scale)
+        self._setup_out(width, left["heads"] * left["vdim"], right["heads"] * right["vdim"], dtype,
+                        device)
+
+    def forward(self, xb: torch.Tensor, md: AttentionMetadata, cache):
+        """cache: (PagedKVRows of the left mixer, DeltaState of the right one)."""
+        kv, state = cache
+        rows = self.right.prepare(self.proj(xb, defer_reduce=True), md, state,
+                                  self.left.attn_prep(kv))
+        heads, lo, ro = self._heads(xb)
+        self.left.attend_prepared(rows.attn_q, rows.attn_gate, md, kv, out=lo)
+        self.right.attend(rows, md, state, out=ro)
         # may return gemm.SplitK: the layer's boundary step reduces it
         return gemm.linear(heads, self.o, defer_reduce=True)
 

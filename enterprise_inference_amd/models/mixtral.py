@@ -220,15 +220,16 @@ class UngatedMLP(nn.Module):
 
     def forward(self, x, pre=None):
         from ..ops import activation, gemm
-        from ..ops.gemm import SplitK, SplitKSlice
+        from ..ops.gemm import SplitKSlice
         if pre is None:
-            pre = gemm.linear(x, self.up.weight, defer_reduce=self.defer and self.kind == "xielu")
+            pre = gemm.linear(x, self.up.weight, defer_reduce=self.defer)
         if self.kind == "relu2":
             if isinstance(pre, SplitKSlice):
                 pre = pre.dense(self.down.weight.dtype)
-            elif isinstance(pre, SplitK):
-                pre = pre.materialize()
-            return self.down(activation.relu2(pre.contiguous()))
+            z = activation.relu2(pre, self.down.weight.dtype)
+            if not self.defer:
+                return self.down(z)
+            return gemm.linear(z, self.down.weight, defer_reduce=True)
         z = activation.xielu(pre, self.act)
         return gemm.linear(z, self.down.weight, defer_reduce=self.defer)
 

@@ -56,15 +56,27 @@ def activation(x: torch.Tensor, act: str) -> torch.Tensor:
     return out
 
 
-def relu2(x: torch.Tensor) -> torch.Tensor:
-    """Squared ReLU, max(x, 0)^2 (bf16 or fp32)."""
-    if not (use_hip(x) and x.is_contiguous() and x.dtype in (torch.bfloat16, torch.float32)):
+def relu2(x, dtype=None) -> torch.Tensor:
+    """Squared ReLU, max(x, 0)^2 (bf16 or fp32), of a tensor with a contiguous last dim or of a
+    ``gemm.SplitK`` (fp32 partial sums of the up-projection, summed here; ``dtype``: the output's,
+    default bf16)."""
+    from .gemm import SplitK
+    if isinstance(x, SplitK):
+        dt = dtype or torch.bfloat16
+        if x.part.is_cuda and x.bias is None and x.N % 4 == 0 and x.part.is_contiguous():
+            out = torch.empty(x.M, x.N, dtype=dt, device=x.part.device)
+            check(lib().eia_relu2(None, 0, ptr(x.part), x.sk, ptr(out), x.N, x.M, x.N,
+                                  1 if dt == torch.bfloat16 else 0, stream(out)), "relu2")
+            return out
+        x = (x.part.sum(0) + (x.bias.float() if x.bias is not None else 0.0)).to(dt)
+    if not (use_hip(x) and x.stride(-1) == 1 and x.dtype in (torch.bfloat16, torch.float32)):
         r = torch.relu(x.float())
         return (r * r).to(x.dtype)
-    out = torch.empty_like(x)
-    check(lib().eia_relu2(ptr(out), ptr(x), x.numel(), 1 if x.dtype == torch.bfloat16 else 0,
-                          stream(x)), "relu2")
-    return out
+    x2 = x if x.dim() == 2 else x.reshape(-1, x.shape[-1])
+    out = torch.empty(x2.shape, dtype=x.dtype, device=x.device)
+    check(lib().eia_relu2(ptr(x2), x2.stride(0), None, 0, ptr(out), out.stride(0), x2.shape[0],
+                          x2.shape[1], 1 if x.dtype == torch.bfloat16 else 0, stream(x)), "relu2")
+    return out.view(x.shape)
 
 
 def xielu(x, pq: torch.Tensor) -> torch.Tensor:

@@ -123,15 +123,16 @@ class ChunkPlan:
         return self.rows * heads * (0.0072 if wide else 0.0052) < serial
 
 
-def chunk_plan(host_lens, device) -> Optional["ChunkPlan"]:
-    """The chunk list of a step whose sequences own ``host_lens`` rows each (batch order), or
-    None when no sequence is long enough for the chunk-parallel form to pay."""
-    if not host_lens or max(host_lens) < CHUNK_MIN_ROWS:
+def chunk_plan(host_lens, device, chunk: int = CHUNK, min_rows: int = CHUNK_MIN_ROWS,
+               row0: int = 0) -> Optional["ChunkPlan"]:
+    """The chunk list of a step whose sequences own ``host_lens`` rows each (batch order, from row
+    ``row0`` on), or None when no sequence is long enough for the chunk-parallel form to pay."""
+    if not host_lens or max(host_lens) < min_rows:
         return None
-    chunks, first, row = [], [0], 0
+    chunks, first, row = [], [0], row0
     for s, n in enumerate(host_lens):
-        for lo in range(0, n, CHUNK):
-            chunks += [s, row + lo, min(CHUNK, n - lo), 0]
+        for lo in range(0, n, chunk):
+            chunks += [s, row + lo, min(chunk, n - lo), 0]
         row += n
         first.append(len(chunks) // 4)
     return ChunkPlan(torch.tensor(chunks, dtype=torch.int32, device=device).view(-1, 4),

@@ -13,8 +13,9 @@ softmax denominator of map m also holds ``exp(sink[m])``, a term without key or 
 ``spec.cap`` > 0 soft-caps the scores, ``cap * tanh(s / cap)``.  With ``spec.talk_post`` the matrix
 ``talk`` mixes the softmax WEIGHTS across the heads instead of the scores (each head's mixed
 weights meet its own kv head's values); its matrix-core form is csrc/kernels/head_mix_attention.hip.
-``spec.epilogue`` 0 multiplies the heads by ``sigmoid(gate)`` and by ``spec.post``; 1 combines
-a head's two maps as ``a1 - lam*a2``, divides by the root mean square over the head and scales.
+``spec.epilogue`` 0 multiplies the heads by ``sigmoid(gate)`` (a value per column, or one per head
+with ``spec.gate_heads``) and by ``spec.post``; 1 combines a head's two maps as ``a1 - lam*a2``,
+divides by the root mean square over the head and scales.
 
 A step's rows are [decode rows (1 per sequence) | prefill chunks]; both parts read the cache
 after ``qk_norm_cache`` wrote this step's rows, so chunked prompts need no special path.
@@ -59,6 +60,7 @@ class WindowSpec:
     sink: Optional[torch.Tensor] = None     # [H*P], exp(sink) joins the softmax denominator
     cap: float = 0.0                # > 0: soft cap on the scores
     talk_post: bool = False         # ``talk`` mixes the softmax weights, not the scores
+    gate_heads: bool = False        # the gate is one number per head, not one per value column
 
 
 def build_work(q_lens: List[int], qblock: int) -> List[int]:
@@ -459,7 +461,8 @@ def _ref_rows(q, k_cache, v_cache, block_table, positions, gate, spec: WindowSpe
         if spec.epilogue == 0:
             o = a[:, 0].reshape(H * Dv) * spec.post
             if gate is not None:
-                o = o * torch.sigmoid(gate[row].float())
+                gv = torch.sigmoid(gate[row].float())
+                o = o * (gv.repeat_interleave(Dv) if spec.gate_heads else gv)
         else:
             o = a[:, 0] - float(spec.lam[0]) * a[:, 1]
             o = (_rms(o, spec.eps) * spec.post).reshape(H * Dv)
@@ -470,7 +473,8 @@ def _ref_rows(q, k_cache, v_cache, block_table, positions, gate, spec: WindowSpe
 def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, md,
                      spec: WindowSpec, gate: Optional[torch.Tensor] = None,
                      out: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """q [T, H*P*D] (normed; contiguous last dim), gate [T, H*Dv] before the sigmoid or None ->
+    """q [T, H*P*D] (normed; contiguous last dim), gate [T, H*Dv] ([T, H] with ``spec.gate_heads``)
+    before the sigmoid or None ->
     [T, H*Dv] in q's dtype.  ``md`` is the step's AttentionMetadata.  ``out``: a [T, H*Dv] view
     (contiguous last dim; the columns of a wider row that another mixer shares) to write into."""
     T = q.shape[0]
@@ -500,7 +504,8 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
             and v_cache.shape[2] == k_cache.shape[1],
             "window_attention: layout")
     require(gate is None or (gate.dtype == q.dtype and gate.stride(1) == 1 and
-                             gate.shape[1] >= H * Dv), "window_attention: gate layout")
+                             gate.shape[1] >= (H if spec.gate_heads else H * Dv)),
+            "window_attention: gate layout")
     require(md.positions.dtype == torch.int32, "positions int32")
     require(spec.weights in (0, 1) and (spec.weights == 0 or (spec.talk is None and P == 1)),
             "window_attention: sigmoid weights come without head mixing or map pairs")
@@ -547,7 +552,7 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
                 ptr(o), o.stride(0), H, spec.kv_heads, P, D, Dv, bs, spec.window, spec.keep,
                 spec.epilogue, ptr(spec.lam), float(spec.eps), float(spec.post), spec.weights,
                 ptr(spec.bias), NP, ptr(pa), ptr(pm), ptr(spec.sink), float(spec.cap),
-                stream(q)), "window_attn_mfma")
+                1 if spec.gate_heads else 0, stream(q)), "window_attn_mfma")
             return
         check(lib().eia_window_attn(
             ptr(qa), qa.stride(0), ptr(k_cache), ptr(v_cache), ptr(bt), bt.stride(0),
@@ -556,7 +561,7 @@ def window_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tens
             o.stride(0), H, spec.kv_heads, P, D, Dv, bs, spec.window, spec.keep, qb,
             spec.epilogue, ptr(spec.lam), float(spec.eps), float(spec.post), spec.weights,
             ptr(spec.bias), ptr(spec.sink), float(spec.cap), 1 if spec.talk_post else 0,
-            1 if bf else 0, stream(q)), "window_attn")
+            1 if spec.gate_heads else 0, 1 if bf else 0, stream(q)), "window_attn")
 
     if nd:
         launch(0, nd, md.decode_block_tables, md.decode_seq_lens, None, None, 1)
