@@ -68,15 +68,18 @@ def parse():
                     help="design: prefill / decode throughput of a layer-list design beside the "
                          "closest existing decoder at equal layer sizes (benchmarks/design_bench.py)")
     ap.add_argument("--design", default="sekolorn",
-                    choices=["sekolorn", "vedadra", "gapidra", "daburax", "borosun"],
+                    choices=["sekolorn", "vedadra", "gapidra", "daburax", "borosun", "vugelix"],
                     help="design mode: sekolorn beside a Mixtral-style decoder, vedadra / gapidra "
                          "beside a Mistral-style decoder (sliding-window GQA attention + gated "
-                         "MLP), daburax beside sekolorn, or borosun beside gapidra")
+                         "MLP), daburax beside sekolorn, borosun beside gapidra, or vugelix "
+                         "beside daburax and borosun")
     ap.add_argument("--design-sizes", default=None,
                     help="comma list; sekolorn: s, s6 (m, l: gated), default s,s6; "
                          "vedadra: vs, vm, default vs,vm; gapidra: gs, gm, default gs,gm; "
-                         "daburax: ds, dm, default ds,dm; borosun: bs, bm, default bs,bm")
-    ap.add_argument("--design-models", default="sekolorn,mixtral,vedadra,mistral,gapidra,daburax,borosun",
+                         "daburax: ds, dm, default ds,dm; borosun: bs, bm, default bs,bm; "
+                         "vugelix: us, um, default us,um")
+    ap.add_argument("--design-models",
+                    default="sekolorn,mixtral,vedadra,mistral,gapidra,daburax,borosun,vugelix",
                     help="which of the two engines to run (profiling one of them alone)")
     ap.add_argument("--design-kernels", action="store_true",
                     help="design mode: time the design's attention / scan kernels beside the "

@@ -23,6 +23,13 @@ per-layer token input; head-mixed full attention behind short convolutions, soft
 attention, gated linear attention) beside Gapidra, the closest existing design (parallel
 sublayers on one norm, window attention, dense feed-forward), at equal width, depth, heads, head
 size, window and ff.
+``--design vugelix`` runs the Vugelix design (hyper-connected residual streams; in every layer a
+soft-capped window attention beside a gated delta rule; dense squared-ReLU feed-forward) beside
+Daburax, the closest existing design (the same streams, attention beside a gated matrix memory),
+with every Daburax layer a parallel one, at equal width, depth, streams, heads and head sizes; Daburax
+has no dense feed-forward: its two routed and one shared gated experts of 2/9 ff each do a token the
+same feed-forward work.  Borosun (dense feed-forward, window attention and gated
+linear attention in separate layers) at the same width, heads and ff is the third row.
 Prefill: ``--design-prompts`` prompts of ``--design-prompt-len`` tokens, one sampled token each.
 Decode: ``--design-users`` sequences of 128 prompt tokens generating ``--design-gen`` tokens; the
 decode rate is the extra tokens over the extra time against the same run with one token.
@@ -199,6 +206,44 @@ def borosun_config(z: dict) -> dict:
             "layers": [att, att2, gla] * (z["layers"] // 3)}
 
 
+USIZES = {
+    # Borosun's sizes, the recurrent side's heads (q / k heads: half as many), streams
+    "us": dict(BSIZES["bs"], rheads=8, streams=4),
+    "um": dict(BSIZES["bm"], rheads=16, streams=4),
+}
+
+
+def vugelix_config(z: dict) -> dict:
+    H, G, D, R = z["heads"], z["kv_heads"], z["dim"], z["rheads"]
+    layer = {"type": "parallel", "mlp": {"kind": "dense", "ff": z["ff"]},
+             "mixer": {"left": {"heads": H, "kv_heads": G, "dim": D, "vdim": D, "scale": D ** -0.5,
+                                "softcap": 30.0, "rot": {"base": 1e5, "dims": D // 2},
+                                "mask": {"size": z["window"]}},
+                       "right": {"heads": R, "kv_heads": R // 2, "dim": D, "vdim": D, "conv": 4},
+                       "left_scale": 1.0, "right_scale": 1.0}}
+    return {"architecture": "Vugelix", "vocab": z["vocab"], "width": z["width"],
+            "norm": {"eps": 1e-6}, "streams": z["streams"], "logit_scale": 0.5,
+            "embedding": {"scale": z["width"] ** 0.5}, "layers": [layer] * z["layers"]}
+
+
+def daburax_like(z: dict) -> dict:
+    """Daburax at a Vugelix size: parallel layers only; the feed-forward work of a token (two routed
+    experts and the shared one, three matrices each) is that of two matrices of ff rows."""
+    ff = -(-z["ff"] * 2 // 9 // 128) * 128
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "shared": {"ff": ff},
+           "router": {"experts": 4, "top": 2, "groups": {"count": 1, "keep": 1}}}
+    H, D = z["heads"], z["dim"]
+    layer = {"type": "parallel", "mlp": mlp,
+             "mixer": {"left": {"heads": H, "kv_heads": z["kv_heads"], "dim": D, "vdim": D,
+                                "scale": D ** -0.5, "rot": {"base": 1e5, "dims": D // 2},
+                                "mask": {"size": z["window"]}},
+                       "right": {"heads": z["rheads"], "dim": D, "vdim": D, "gate_cap": 15.0},
+                       "left_scale": 1.0, "right_scale": 1.0}}
+    return {"architecture": "Daburax", "vocab": z["vocab"], "width": z["width"],
+            "norm": {"eps": 1e-6}, "streams": z["streams"],
+            "embedding": {"scale": z["width"] ** 0.5}, "layers": [layer] * z["layers"]}
+
+
 def sekolorn_like(z: dict) -> dict:
     """Sekolorn at a Daburax size: same width, depth, heads, experts, top-k and expert ff."""
     return sekolorn_config(dict(width=z["width"], layers=z["layers"], heads=z["heads"], dim=64,
@@ -259,7 +304,7 @@ def run(a) -> int:
     design = getattr(a, "design", "sekolorn")
     vedadra = design == "vedadra"
     default = {"vedadra": "vs,vm", "gapidra": "gs,gm", "daburax": "ds,dm",
-               "borosun": "bs,bm"}.get(design, "s,s6")
+               "borosun": "bs,bm", "vugelix": "us,um"}.get(design, "s,s6")
     for name in (a.design_sizes or default).split(","):
         if name in GATED:
             raise SystemExit(f"design size {name!r} is switched off (see GATED in "
@@ -271,6 +316,10 @@ def run(a) -> int:
             other = ("Sekolorn", sekolorn_like(z)) if name == "ds" else \
                 ("Mixtral-style", mixtral_config(z))
             pair = (("Daburax", daburax_config(z)), other)
+        elif design == "vugelix":
+            z = USIZES[name]
+            pair = (("Vugelix", vugelix_config(z)), ("Daburax", daburax_like(z)),
+                    ("Borosun", borosun_config(z)))
         elif design == "borosun":
             z = BSIZES[name]
             pair = (("Borosun", borosun_config(z)), ("Gapidra", gapidra_config(z)))
@@ -328,6 +377,8 @@ def kernel_rates(a) -> int:
         return daburax_kernel_rates(a)
     if getattr(a, "design", "sekolorn") == "borosun":
         return borosun_kernel_rates(a)
+    if getattr(a, "design", "sekolorn") == "vugelix":
+        return vugelix_kernel_rates(a)
     from enterprise_inference_amd.ops import attention as A
     from enterprise_inference_amd.ops import latent_attention as LA
     from enterprise_inference_amd.ops import wkv as WK
@@ -976,6 +1027,163 @@ def borosun_kernel_rates(a) -> int:
             t = _time(fn)
             rows.append({"kernel": label, "width": W, "rows": Tn, "ms": t * 1e3,
                          "GBps": Tn * nbytes / t / 1e9})
+    for r in rows:
+        print(json.dumps(r), flush=True)
+    print(json.dumps({"metric": "design_kernel_rates", "rows": rows}), flush=True)
+    return 0
+
+
+def vugelix_kernel_rates(a) -> int:
+    """Achieved rates of the Vugelix kernels beside their like kernels at equal heads and lengths: the
+    gated delta scan (both forms) beside the gated linear scan of Daburax's matrix memory and the
+    fixed-decay one (tokens/s, at decode state bytes/s); soft-capped window attention with a unit sink
+    and head gates beside the same family with a learned sink (Daburax), causal and windowed; the
+    prep launch of both sides beside the attention-only and convolution preps (bytes/s); the boundary
+    over four streams; the squared ReLU beside the gated activation.  One JSON line per kernel."""
+    import torch
+
+    from enterprise_inference_amd.ops import activation as AC
+    from enterprise_inference_amd.ops import attention as A
+    from enterprise_inference_amd.ops import delta_scan as DS
+    from enterprise_inference_amd.ops import gemm as GM
+    from enterprise_inference_amd.ops import linear_scan as LS
+    from enterprise_inference_amd.ops import norm as N
+    from enterprise_inference_amd.ops import window_attention as WA
+    from enterprise_inference_amd.ops.rotary import rotary_frequencies
+
+    dev, bf = "cuda", torch.bfloat16
+    rows = []
+    i32 = lambda v: torch.tensor(v, dtype=torch.int32, device=dev)
+    bs, win, D = 128, 1024, 128
+
+    def meta(nseq, per):
+        """A step of nseq fresh prompts of ``per`` tokens, or (per 1) nseq decode rows at 4096."""
+        T = nseq * per
+        ar = torch.arange(T, dtype=torch.int32, device=dev)
+        slots = torch.arange(nseq, dtype=torch.int32, device=dev)
+        if per == 1:
+            L = 4096
+            bt = torch.arange(nseq * L // bs, dtype=torch.int32, device=dev).view(nseq, -1)
+            return A.AttentionMetadata(
+                num_decode=nseq, num_prefill_tokens=0, slot_mapping=bt[:, -1] * bs + bs - 1,
+                positions=torch.full((nseq,), L - 1, dtype=torch.int32, device=dev),
+                decode_block_tables=bt, decode_seq_lens=i32([L] * nseq), num_seqs=nseq,
+                seq_slots=slots), nseq * L // bs
+        cu = torch.arange(0, T + 1, per, dtype=torch.int32, device=dev)
+        wl = A.build_prefill_work([per] * nseq, WA.MFMA_QB)
+        return A.AttentionMetadata(
+            num_decode=0, num_prefill_tokens=T, slot_mapping=ar, positions=ar % per,
+            prefill_block_tables=torch.arange(T // bs, dtype=torch.int32, device=dev).view(nseq, -1),
+            prefill_seq_lens=i32([per] * nseq), prefill_cu_q=cu, prefill_q_lens=[per] * nseq,
+            prefill_work=i32(wl), prefill_n_work=len(wl) // 2, prefill_qblock=WA.MFMA_QB,
+            num_seqs=nseq, seq_slots=slots, seq_cu=cu), T // bs
+
+    # ---- both sides of a layer at the two bench sizes (and the scan at 64-wide heads)
+    for H, G, R, Dr in ((8, 2, 8, 128), (16, 4, 16, 128), (16, 4, 32, 64)):
+        K = R // 2
+        inv, _ = rotary_frequencies(D // 2, 1e5, None, dev)
+        offs, n = {}, (H + 2 * G) * D + H
+        for name, c in (("q", K * Dr), ("k", K * Dr), ("v", R * Dr), ("g", R * Dr), ("b", R), ("a", R)):
+            n = -(-n // 8) * 8
+            offs[name] = n
+            n += c
+        n = -(-n // 64) * 64
+        cw = lambda c: (torch.randn(c, 4, device=dev) * 0.4).to(bf)
+        spec = DS.DeltaSpec(R, K, Dr, Dr, 4, cw(K * Dr), cw(K * Dr), cw(R * Dr),
+                            torch.full((R,), 0.5, device=dev), torch.full((R,), -3.0, device=dev),
+                            Dr ** -0.5, 1.0, 1e-6)
+        nw = torch.ones(Dr, device=dev).to(bf)
+        for nseq, per in ((1, 4096), (1, 2048), (4, 2048), (16, 128), (64, 1)):
+            md, nb = meta(nseq, per)
+            T = nseq * per
+            fused = (torch.randn(T, n, device=dev) * 0.5).to(bf)
+            st = DS.DeltaState.allocate(nseq, spec, bf, dev)
+            kc = torch.randn(nb, bs, G * D, device=dev).to(bf)
+            vc = torch.randn(nb, G * D, bs, device=dev).to(bf)
+            ap = DS.AttnPrep(0, H * D, (H + G) * D, WA.PrepSpec(H, G, D, D, inv, D // 2, True), kc, vc,
+                             (H + 2 * G) * D, H)
+            t = _time(lambda: DS.delta_prep(fused, offs, spec, st, md, ap))
+            moved = T * (2 * (n + (H + 2 * G) * D) + 4 * (2 * K + R) * Dr)
+            rows.append({"kernel": "delta_prep (both sides)", "heads": H, "rheads": R, "rows": T,
+                         "ms": t * 1e3, "GBps": moved / t / 1e9})
+            r = DS.delta_prep(fused, offs, spec, st, md, ap)
+            if Dr == D:
+                WA.qk_rope_cache(fused, 0, H * D, (H + G) * D, H, G, D, G * D, None, None, inv,
+                                 D // 2, True, 1.0, md.positions, kc, vc, md.slot_mapping, 1e-6)
+                t = _time(lambda: WA.qk_rope_cache(
+                    fused, 0, H * D, (H + G) * D, H, G, D, G * D, None, None, inv, D // 2, True, 1.0,
+                    md.positions, kc, vc, md.slot_mapping, 1e-6))
+                rows.append({"kernel": "qk_rope_cache (attention side alone)", "heads": H, "rows": T,
+                             "ms": t * 1e3, "GBps": T * (H + 2 * G) * D * 4 / t / 1e9})
+            forms = [("token by token", False)] + ([("chunk-parallel", True)] if per > 1 else [])
+            for form, force in forms:
+                DS.FORCE_CHUNKED = force
+                plan = DS.prefill_plan(md, torch.device(dev)) if force else None
+                t = _time(lambda: DS.delta_scan(r, spec, st, md, nw, None, plan))
+                rows.append({"kernel": f"delta_scan ({form})", "heads": R, "kv_heads": K, "dim": Dr,
+                             "seqs": nseq, "tokens_per_seq": per, "ms": t * 1e3,
+                             "tokens_per_s": T / t,
+                             "state_GBps": nseq * R * Dr * Dr * 4 * 2 / t / 1e9})
+            DS.FORCE_CHUNKED = None
+            x = (torch.randn(T, 4 * R * Dr + 2 * R, device=dev) * 0.3).to(bf)
+            for mode in ("exp_gates", "decay"):
+                sp = LS.ScanSpec(R, Dr, Dr, mode, decay=torch.full((R,), 0.97, device=dev), cap=15.0,
+                                 kscale=Dr ** -0.5, gate_act="silu" if mode == "decay" else "sigmoid",
+                                 eps=1e-5)
+                ls = LS.ScanState.allocate(nseq, sp, dev)
+                for form, force in forms:
+                    LS.FORCE_CHUNKED = force
+                    plan = LS.chunk_plan([per] * nseq, dev) if force else None
+                    t = _time(lambda: LS.linear_scan(
+                        x, 0, R * Dr, 2 * R * Dr, 3 * R * Dr, sp, ls, md.seq_slots, md.seq_cu, nseq,
+                        md.positions, None, None, 4 * R * Dr, 4 * R * Dr + R, plan=plan))
+                    rows.append({"kernel": f"linear_scan ({mode}, {form})", "heads": R, "dim": Dr,
+                                 "seqs": nseq, "tokens_per_seq": per, "ms": t * 1e3,
+                                 "tokens_per_s": T / t,
+                                 "state_GBps": nseq * R * Dr * Dr * 4 * 2 / t / 1e9})
+                LS.FORCE_CHUNKED = False
+            if Dr != D or (nseq, per) not in ((1, 4096), (64, 1)):
+                continue
+            q = torch.randn(T, H * D, device=dev).to(bf)
+            gate = torch.randn(T, H, device=dev).to(bf)
+            mult = torch.full((H,), D ** -0.5, device=dev)
+            mk = lambda **kw: WA.WindowSpec(H, G, 1, D, D, kw.pop("window", 0), 0, mult=mult,
+                                            sink=torch.zeros(H, device=dev), **kw)
+            wpairs = per * win - win * (win - 1) // 2
+            for label, ws, g_, pairs, keys in (
+                    ("soft cap, unit sink, head gate, window", mk(cap=30.0, window=win,
+                                                                  gate_heads=True), gate, wpairs, win),
+                    ("learned sink, window", mk(window=win), None, wpairs, win),
+                    ("learned sink, causal", mk(), None, per * (per + 1) // 2, 4096)):
+                t = _time(lambda: WA.window_attention(q, kc, vc, md, ws, g_))
+                row = {"kernel": f"attention {'prefill' if per > 1 else 'decode'} ({label})",
+                       "heads": H, "kv_heads": G, "dim": D, "ms": t * 1e3}
+                if per > 1:
+                    row["tflops"] = 4.0 * D * H * pairs / t / 1e12
+                else:
+                    row["cache_GBps"] = nseq * keys * G * 2 * D * 2 / t / 1e9
+                rows.append(row)
+    # ---- boundary and activation
+    for W, ff in ((1024, 4096), (2048, 8192)):
+        for Tn in (8192, 32):
+            X = torch.randn(Tn, 4, W, device=dev)
+            y = torch.randn(Tn, W, device=dev).to(bf)
+            w1, mix, ones = torch.ones(W, device=dev).to(bf), torch.eye(4, device=dev), \
+                torch.ones(4, device=dev)
+            t = _time(lambda: N.hyper_step(X, 1e-5, y, mix, ones, 1.0, ones, w1, 0.0))
+            rows.append({"kernel": "hyper_step (4 streams)", "width": W, "rows": Tn, "ms": t * 1e3,
+                         "GBps": Tn * W * (2 * 4 * 4 + 2 + 2) / t / 1e9})
+            u = torch.randn(Tn, 2 * ff, device=dev).to(bf)
+            t = _time(lambda: AC.relu2(u[:, :ff]))
+            rows.append({"kernel": "relu2", "ff": ff, "rows": Tn, "ms": t * 1e3,
+                         "GBps": Tn * ff * 4 / t / 1e9})
+            t = _time(lambda: AC.silu_and_mul(u))
+            rows.append({"kernel": "silu_and_mul", "ff": ff, "rows": Tn, "ms": t * 1e3,
+                         "GBps": Tn * ff * 6 / t / 1e9})
+        part = GM.SplitK(torch.randn(4, 32, ff, device=dev), 4, 32, ff)
+        t = _time(lambda: AC.relu2(part))
+        rows.append({"kernel": "relu2 (split-K partials)", "ff": ff, "rows": 32, "ms": t * 1e3,
+                     "GBps": 32 * ff * 18 / t / 1e9})
     for r in rows:
         print(json.dumps(r), flush=True)
     print(json.dumps({"metric": "design_kernel_rates", "rows": rows}), flush=True)

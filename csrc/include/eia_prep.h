@@ -46,8 +46,13 @@ EIA_DEV float prep_load(const PrepRows& p, long r, int col) {     // as the acti
   if (p.x) return ld_f32<T>((const T*)p.x + r * p.ld, col);
   float v = p.bias ? ld_f32<T>((const T*)p.bias, col) : 0.f;
   const float* q = p.part + r * p.ld + col;
-#pragma unroll 4
-  for (int z = 0; z < p.sk; ++z) v += q[z * p.pstride];
+  for (int z0 = 0; z0 < p.sk; z0 += 4) {               // four partials in flight
+    float u[4];
+#pragma unroll
+    for (int z = 0; z < 4; ++z) u[z] = q[min(z0 + z, p.sk - 1) * p.pstride];
+#pragma unroll
+    for (int z = 0; z < 4; ++z) v += z0 + z < p.sk ? u[z] : 0.f;
+  }
   return (float)(T)v;
 }
 
@@ -55,15 +60,16 @@ EIA_DEV float prep_load(const PrepRows& p, long r, int col) {     // as the acti
 // head's columns start at col0 in the fused row and at channel c0 of its weights cw [., taps],
 // taps <= TAPS; S: the head's first channel in the sequence's history slot (rows of ST), null: no
 // slot.
-template <typename T, int TAPS, int NE>
+template <typename T, int TAPS, int NE, int NR>
 EIA_DEV void prep_conv(const PrepRows& rows, const PrepRun& run, int pos0, const T* cw, int c0,
                        int col0, T* S, int ST, const int (&da)[NE], const int (&db)[NE],
-                       const bool (&oka)[NE], const bool (&okb)[NE], float (&ua)[NE][QP_ROWS],
-                       float (&ub)[NE][QP_ROWS], const int taps = TAPS) {
+                       const bool (&oka)[NE], const bool (&okb)[NE], float (&ua)[NE][NR],
+                       float (&ub)[NE][NR], const int taps = TAPS) {
   constexpr int NH = TAPS > 1 ? TAPS - 1 : 1;
   const int j0 = TAPS - taps;                          // unused oldest taps
-  auto load = [&](long r, int d, bool ok) -> float {
-    return ok ? prep_load<T>(rows, r, col0 + d) : 0.f;
+  auto load = [&](long r, int d, bool ok) -> float {            // (address clamped, no branch)
+    const float v = prep_load<T>(rows, r, col0 + (ok ? d : 0));
+    return ok ? v : 0.f;
   };
   if constexpr (TAPS > 1) {
 #pragma unroll
@@ -71,8 +77,11 @@ EIA_DEV void prep_conv(const PrepRows& rows, const PrepRun& run, int pos0, const
       float ha[NH], hb[NH], wa[TAPS], wb[TAPS];
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) {
-        wa[j] = oka[e] && j >= j0 ? ld_f32<T>(cw, (long)(c0 + da[e]) * taps + j - j0) : 0.f;
-        wb[j] = okb[e] && j >= j0 ? ld_f32<T>(cw, (long)(c0 + db[e]) * taps + j - j0) : 0.f;
+        const int jj = j >= j0 ? j - j0 : 0;
+        wa[j] = ld_f32<T>(cw, (long)(c0 + (oka[e] ? da[e] : 0)) * taps + jj);
+        wb[j] = ld_f32<T>(cw, (long)(c0 + (okb[e] ? db[e] : 0)) * taps + jj);
+        if (j < j0 || !oka[e]) wa[j] = 0.f;
+        if (j < j0 || !okb[e]) wb[j] = 0.f;
       }
       // the TAPS - 1 values before the run: earlier rows of the portion, or the slot, or zeros
 #pragma unroll
@@ -84,8 +93,8 @@ EIA_DEV void prep_conv(const PrepRows& rows, const PrepRun& run, int pos0, const
           va = load(run.row - back, da[e], oka[e]);
           vb = load(run.row - back, db[e], okb[e]);
         } else if (pos0 >= back && S) {
-          if (oka[e]) va = ld_f32<T>(S, (long)(j - j0) * ST + da[e]);
-          if (okb[e]) vb = ld_f32<T>(S, (long)(j - j0) * ST + db[e]);
+          va = ld_f32<T>(S, (long)(j - j0) * ST + (oka[e] ? da[e] : 0));
+          vb = ld_f32<T>(S, (long)(j - j0) * ST + (okb[e] ? db[e] : 0));
         }
         ha[j] = va;
         hb[j] = vb;
@@ -109,7 +118,7 @@ EIA_DEV void prep_conv(const PrepRows& rows, const PrepRun& run, int pos0, const
         }
       }
 #pragma unroll
-      for (int i = QP_ROWS - 1; i >= 0; --i) {         // last row first: earlier rows still hold u
+      for (int i = NR - 1; i >= 0; --i) {         // last row first: earlier rows still hold u
         float ya = 0.f, yb = 0.f;
 #pragma unroll
         for (int j = 0; j < TAPS; ++j) {
@@ -127,7 +136,7 @@ EIA_DEV void prep_conv(const PrepRows& rows, const PrepRun& run, int pos0, const
       const float wa = oka[e] ? ld_f32<T>(cw, c0 + da[e]) : 0.f;
       const float wb = okb[e] ? ld_f32<T>(cw, c0 + db[e]) : 0.f;
 #pragma unroll
-      for (int i = 0; i < QP_ROWS; ++i) {
+      for (int i = 0; i < NR; ++i) {
         ua[e][i] *= wa;
         ub[e][i] *= wb;
       }
@@ -135,8 +144,8 @@ EIA_DEV void prep_conv(const PrepRows& rows, const PrepRun& run, int pos0, const
   }
 }
 
-// One unit (head of q, k or v) of a run.
-template <typename T, int TAPS, int NE>
+// One unit (head of q, k or v) of a run of up to NR rows.
+template <typename T, int TAPS, int NE, int NR = QP_ROWS>
 EIA_DEV void qkv_prep_unit(const QkvPrepArgs& a, const PrepRun& run, int unit) {
   const int lane = threadIdx.x & 63;
   const int n = run.n;
@@ -165,29 +174,30 @@ EIA_DEV void qkv_prep_unit(const QkvPrepArgs& a, const PrepRun& run, int unit) {
     fr[e] = rot[e] ? a.inv_freq[s] : 0.f;
   }
   const PrepRows rows{a.x, a.ld, a.part, a.sk, a.pstride, a.bias};
-  auto load = [&](long r, int d, bool ok) -> float {
-    return ok ? prep_load<T>(rows, r, col0 + d) : 0.f;
+  auto load = [&](long r, int d, bool ok) -> float {            // (address clamped, no branch)
+    const float v = prep_load<T>(rows, r, col0 + (ok ? d : 0));
+    return ok ? v : 0.f;
   };
-  float ua[NE][QP_ROWS], ub[NE][QP_ROWS];
+  float ua[NE][NR], ub[NE][NR];
 #pragma unroll
   for (int e = 0; e < NE; ++e)
 #pragma unroll
-    for (int i = 0; i < QP_ROWS; ++i) {
-      ua[e][i] = i < n ? load(row + i, da[e], oka[e]) : 0.f;
-      ub[e][i] = i < n ? load(row + i, db[e], okb[e]) : 0.f;
+    for (int i = 0; i < NR; ++i) {
+      ua[e][i] = load(row + min(i, n - 1), da[e], oka[e]);      // (rows past the run: unused)
+      ub[e][i] = load(row + min(i, n - 1), db[e], okb[e]);
     }
   const int pos0 = a.positions[row];
   if constexpr (TAPS > 1) {
     const int slot = a.seq_slots[run.seq];
-    prep_conv<T, TAPS, NE>(rows, run, pos0, cw, c0, col0,
+    prep_conv<T, TAPS, NE, NR>(rows, run, pos0, cw, c0, col0,
                            slot >= 0 ? (T*)a.state + (long)slot * (TAPS - 1) * ST + st0 : nullptr,
                            ST, da, db, oka, okb, ua, ub);
   } else if (cw) {
-    prep_conv<T, 1, NE>(rows, run, pos0, cw, c0, col0, nullptr, 0, da, db, oka, okb, ua, ub);
+    prep_conv<T, 1, NE, NR>(rows, run, pos0, cw, c0, col0, nullptr, 0, da, db, oka, okb, ua, ub);
   }
   if (isq || isk) {
 #pragma unroll
-    for (int i = 0; i < QP_ROWS; ++i) {
+    for (int i = 0; i < NR; ++i) {
       if (i >= n) break;
       const float pos = (float)(pos0 + i);
       float ss = 0.f;
@@ -225,7 +235,7 @@ EIA_DEV void qkv_prep_unit(const QkvPrepArgs& a, const PrepRun& run, int unit) {
 #pragma unroll
     for (int e = 0; e < NE; ++e)
 #pragma unroll
-      for (int i = 0; i < QP_ROWS; ++i) {
+      for (int i = 0; i < NR; ++i) {
         if (i >= n) break;
         T* f = F + (row + i) * VW + c0;
         if (a.v_mode == 1) {
@@ -239,20 +249,20 @@ EIA_DEV void qkv_prep_unit(const QkvPrepArgs& a, const PrepRun& run, int unit) {
   }
   // eight consecutive tokens of one page: one 16-byte (bf16) or two (fp32) stores per column
   const long s0 = a.slots[row];
-  bool run8 = n == QP_ROWS && s0 >= 0 && s0 % QP_ROWS == 0 && a.bs % QP_ROWS == 0;
+  bool run8 = NR == QP_ROWS && n == QP_ROWS && s0 >= 0 && s0 % QP_ROWS == 0 && a.bs % QP_ROWS == 0;
   if (run8) {
 #pragma unroll
-    for (int i = 1; i < QP_ROWS; ++i) run8 = run8 && a.slots[row + i] == s0 + i;
+    for (int i = 1; i < NR; ++i) run8 = run8 && a.slots[row + i] == s0 + i;
   }
   T* V = (T*)a.vc;
 #pragma unroll
   for (int e = 0; e < NE; ++e) {
     if (run8) {
       const long base = (s0 / a.bs) * VW * a.bs + s0 % a.bs;
-      alignas(16) T ra[QP_ROWS], rb[QP_ROWS];
+      alignas(16) T ra[NR], rb[NR];
 #pragma unroll
-      for (int i = 0; i < QP_ROWS; ++i) { ra[i] = (T)ua[e][i]; rb[i] = (T)ub[e][i]; }
-      constexpr int NV = QP_ROWS * sizeof(T) / 16;
+      for (int i = 0; i < NR; ++i) { ra[i] = (T)ua[e][i]; rb[i] = (T)ub[e][i]; }
+      constexpr int NV = NR * sizeof(T) / 16;
       if (oka[e])
 #pragma unroll
         for (int w = 0; w < NV; ++w)
@@ -266,7 +276,7 @@ EIA_DEV void qkv_prep_unit(const QkvPrepArgs& a, const PrepRun& run, int unit) {
       continue;
     }
 #pragma unroll
-    for (int i = 0; i < QP_ROWS; ++i) {
+    for (int i = 0; i < NR; ++i) {
       if (i >= n) break;
       const long slot = a.slots[row + i];
       if (slot < 0) continue;

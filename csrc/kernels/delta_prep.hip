@@ -31,7 +31,7 @@ struct DeltaPrepArgs {
 EIA_DEV float dl_silu(float z) { return z / (1.0f + expf(-z)); }
 EIA_DEV float dl_softplus(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
 
-template <typename T, int TAPS, int NE>
+template <typename T, int TAPS, int NE, int NR>
 EIA_DEV void delta_prep_unit(const DeltaPrepArgs& a, const PrepRun& run, int unit) {
   const int lane = threadIdx.x & 63, n = run.n;
   const long row = run.row;
@@ -69,7 +69,7 @@ EIA_DEV void delta_prep_unit(const DeltaPrepArgs& a, const PrepRun& run, int uni
   const T* cw = (const T*)(isq ? a.cw_q : isk ? a.cw_k : a.cw_v);
   int da[NE], db[NE];
   bool oka[NE], okb[NE];
-  float ua[NE][QP_ROWS], ub[NE][QP_ROWS];
+  float ua[NE][NR], ub[NE][NR];
 #pragma unroll
   for (int e = 0; e < NE; ++e) {
     da[e] = 2 * (lane + 64 * e);
@@ -77,20 +77,23 @@ EIA_DEV void delta_prep_unit(const DeltaPrepArgs& a, const PrepRun& run, int uni
     oka[e] = da[e] < D;
     okb[e] = db[e] < D;
 #pragma unroll
-    for (int i = 0; i < QP_ROWS; ++i) {
-      ua[e][i] = (i < n && oka[e]) ? prep_load<T>(a.rows, row + i, col0 + da[e]) : 0.f;
-      ub[e][i] = (i < n && okb[e]) ? prep_load<T>(a.rows, row + i, col0 + db[e]) : 0.f;
+    for (int i = 0; i < NR; ++i) {
+      // (addresses clamped, no branches: the loads of a run are in flight together)
+      ua[e][i] = prep_load<T>(a.rows, row + min(i, n - 1), col0 + (oka[e] ? da[e] : 0));
+      ub[e][i] = prep_load<T>(a.rows, row + min(i, n - 1), col0 + (okb[e] ? db[e] : 0));
+      if (!oka[e]) ua[e][i] = 0.f;
+      if (!okb[e]) ub[e][i] = 0.f;
     }
   }
   const int slot = a.taps > 1 ? a.seq_slots[run.seq] : -1;
-  prep_conv<T, TAPS, NE>(a.rows, run, a.positions[row], cw, c0, col0,
+  prep_conv<T, TAPS, NE, NR>(a.rows, run, a.positions[row], cw, c0, col0,
                          slot >= 0 ? (T*)a.state + (long)slot * (a.taps - 1) * ST + st0 : nullptr,
                          ST, da, db, oka, okb, ua, ub, a.taps);
   float* dst = isq ? a.q + row * a.G * a.DP : isk ? a.k + row * a.G * a.DP : a.v + row * a.H * a.VP;
   const long ld = (long)((isq || isk) ? a.G : a.H) * P;
   dst += (long)hh * P;
 #pragma unroll
-  for (int i = 0; i < QP_ROWS; ++i) {
+  for (int i = 0; i < NR; ++i) {
     if (i >= n) break;
     float ss = 0.f;
 #pragma unroll
@@ -110,16 +113,17 @@ EIA_DEV void delta_prep_unit(const DeltaPrepArgs& a, const PrepRun& run, int uni
   }
 }
 
-// The attention mixer's units (w.H + 2 w.G; none when w.H is 0) come first.  TAPS: at least a.taps.
-template <typename T, int TAPS, int NE>
+// The attention mixer's units (w.H + 2 w.G; none when w.H is 0) come first.  TAPS: at least a.taps;
+// NR: rows of a run (1 in decode steps).
+template <typename T, int TAPS, int NE, int NR>
 __global__ void __launch_bounds__(256)
 delta_prep_kernel(const DeltaPrepArgs a, const QkvPrepArgs w, int units) {
   const int unit = blockIdx.y * 4 + (threadIdx.x >> 6), nw = w.H ? w.H + 2 * w.G : 0;
   if (unit >= units) return;
   const PrepRun run = prep_run(a.cu, a.work, a.row_base, blockIdx.x);
   if (run.n <= 0) return;
-  if (unit < nw) qkv_prep_unit<T, 1, NE>(w, run, unit);
-  else delta_prep_unit<T, TAPS, NE>(a, run, unit - nw);
+  if (unit < nw) qkv_prep_unit<T, 1, NE, NR>(w, run, unit);
+  else delta_prep_unit<T, TAPS, NE, NR>(a, run, unit - nw);
 }
 
 // n_items: decode rows (work == nullptr) or prefill runs of QP_ROWS rows.  wH > 0: the attention
@@ -156,8 +160,12 @@ EIA_API int eia_delta_prep(const void* x, long ld, const float* part, int sk, lo
   const int units = 2 * G + H + (g_out ? H : 0) + 1 + (wH ? wH + 2 * wG : 0);
   const dim3 grid(n_items, (units + 3) / 4);
   const bool wide = DP > 128 || VP > 128 || wD > 128 || wDv > 128;
-#define DP_GO(TT, N, NE) \
-  hipLaunchKernelGGL((delta_prep_kernel<TT, N, NE>), grid, dim3(256), 0, st, a, w, units)
+#define DP_GO1(TT, N, NE, NR) \
+  hipLaunchKernelGGL((delta_prep_kernel<TT, N, NE, NR>), grid, dim3(256), 0, st, a, w, units)
+#define DP_GO(TT, N, NE)                                                       \
+  do {                                                                        \
+    if (work) DP_GO1(TT, N, NE, QP_ROWS); else DP_GO1(TT, N, NE, 1);          \
+  } while (0)
 #define DP_SIZES(TT)                                          \
   do {                                                        \
     if (taps <= 4) {                                          \
@@ -169,5 +177,6 @@ EIA_API int eia_delta_prep(const void* x, long ld, const float* part, int sk, lo
   if (is_bf16) DP_SIZES(bf16_t); else DP_SIZES(float);
 #undef DP_SIZES
 #undef DP_GO
+#undef DP_GO1
   EIA_LAUNCH_CHECK();
 }

@@ -30,49 +30,42 @@ struct DeltaArgs {
 };
 
 // Token by token: one workgroup of 256 threads per (sequence, head).  Thread (rg, cg) owns rows
-// rg, rg + RG, ... and V columns of S in registers (RG = 256 / CGP row groups, CGP column groups, a
-// power of two).  Per token one pass over the registers forms S^T k and S^T q of the state BEFORE the
-// token and k . q; with them u = b (v - a S^T k) and o = a S^T q + (k . q) u, so the update needs no
-// second reduction (partial sums of odd and even tokens alternate between two LDS buffers: one
-// barrier per token).  Tokens are staged TC at a time.
+// rg, rg + RG, ... and columns 4 cg .. of S in registers (CGP = 2^LG column groups, RG = 256 / CGP row
+// groups).  Per token one pass over the registers forms S^T k and S^T q of the state BEFORE the
+// token; with them and k . q, u = b (v - a S^T k) and o = a S^T q + (k . q) u, so the update needs no
+// second reduction (the four waves' partial sums of odd and even tokens alternate between two LDS
+// buffers: one barrier per token).  Tokens are staged DS_TC at a time, (k, q) pairs zero past D.
+// vec: 16-byte accesses to the state.
 constexpr int DS_TC = 8;
 
-template <typename T, int V, int RPT>
+template <typename T, int LG, int RPT>
 __global__ void __launch_bounds__(256)
-delta_scan_kernel(DeltaArgs a, int cgp_log2) {
-  extern __shared__ __align__(16) float lds[];
+delta_scan_kernel(DeltaArgs a, int vec) {
+  constexpr int CGP = 1 << LG, RG = 256 >> LG, CW = 4 * CGP, RW = RG * RPT;
+  __shared__ __align__(16) float2 skq[DS_TC][RW];
+  __shared__ __align__(16) float sv[DS_TC][CW], so[DS_TC][CW], sp[2][4][2][CW];
+  __shared__ float dot[DS_TC], sa[DS_TC], sb[DS_TC];
   const int s = blockIdx.x, h = blockIdx.y, tid = threadIdx.x;
   const int slot = a.slots[s];
   if (slot < 0 || (a.seq_lens && a.seq_lens[s] <= 0)) return;
   const int lo = a.cu ? a.cu[s] : s, hi = a.cu ? a.cu[s + 1] : s + 1;
   if (hi <= lo) return;
   const int H = a.H, G = a.G, D = a.D, Dv = a.Dv, DP = a.DP, VP = a.VP, kh = h / (H / G);
-  const int CGP = 1 << cgp_log2, RG = 256 >> cgp_log2;
-  const int cg = tid & (CGP - 1), rg = tid >> cgp_log2, c0 = V * cg;
-  const int np = CGP >= 64 ? RG : 4;                   // partial sums per column
-  const int pi = CGP >= 64 ? rg : tid >> 6;
-  const int PW = 2 * V * CGP + 4;                      // one partial: S^T k, S^T q, k . q
-  float* sq = lds;                                     // [TC][DP]
-  float* sk = sq + DS_TC * DP;
-  float* sv = sk + DS_TC * DP;                         // [TC][V * CGP]
-  float* so = sv + DS_TC * V * CGP;
-  float* sp = so + DS_TC * V * CGP;                    // [2][np][PW]
-  float* sab = sp + 2 * np * PW;                       // [TC] decay, [TC] step size
-  const bool col = c0 < Dv;
+  const int cg = tid & (CGP - 1), rg = tid >> LG, c0 = 4 * cg;
   float* Sg = a.S + ((long)slot * H + h) * D * Dv;
   const bool fresh = a.positions[lo] == 0;
-  float S[RPT][V];
+  f32x4 S[RPT];
 #pragma unroll
   for (int ii = 0; ii < RPT; ++ii) {
     const int i = rg + RG * ii;
-    const bool ok = !fresh && col && i < D;
-    if constexpr (V == 4) {
-      const f32x4 v = ok ? *reinterpret_cast<const f32x4*>(Sg + (long)i * Dv + c0)
-                         : f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll
-      for (int e = 0; e < V; ++e) S[ii][e] = v[e];
+    S[ii] = f32x4{0.f, 0.f, 0.f, 0.f};
+    if (fresh || i >= D || c0 >= Dv) continue;
+    if (vec) {
+      S[ii] = *reinterpret_cast<const f32x4*>(Sg + (long)i * Dv + c0);
     } else {
-      S[ii][0] = ok ? Sg[(long)i * Dv + c0] : 0.f;
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (c0 + e < Dv) S[ii][e] = Sg[(long)i * Dv + c0 + e];
     }
   }
   const T* NW = static_cast<const T*>(a.norm_w);
@@ -82,100 +75,86 @@ delta_scan_kernel(DeltaArgs a, int cgp_log2) {
   for (int base = lo; base < hi; base += DS_TC) {
     const int nt = min(DS_TC, hi - base);
     __syncthreads();                                   // the previous tokens' LDS reads are done
-    for (int idx = tid; idx < nt * DP; idx += 256) {
-      const int t = idx / DP, d = idx - t * DP;
-      const long r = ((long)(base + t) * G + kh) * DP + d;
-      sq[idx] = a.q[r];
-      sk[idx] = a.k[r];
+    for (int idx = tid; idx < nt * RW; idx += 256) {
+      const int t = idx / RW, d = idx % RW;
+      const long r = ((long)(base + t) * G + kh) * DP + min(d, DP - 1);
+      skq[t][d] = d < D ? make_float2(a.k[r], a.q[r]) : make_float2(0.f, 0.f);
     }
-    for (int idx = tid; idx < nt * V * CGP; idx += 256) {
-      const int t = idx / (V * CGP), d = idx - t * V * CGP;
-      sv[idx] = d < Dv ? a.v[((long)(base + t) * H + h) * VP + d] : 0.f;
+    for (int idx = tid; idx < nt * CW; idx += 256) {
+      const int t = idx / CW, d = idx % CW;
+      sv[t][d] = d < Dv ? a.v[((long)(base + t) * H + h) * VP + d] : 0.f;
     }
     if (tid < nt) {
-      sab[tid] = expf(a.la[(long)(base + tid) * H + h]);
-      sab[DS_TC + tid] = a.beta[(long)(base + tid) * H + h];
+      sa[tid] = expf(a.la[(long)(base + tid) * H + h]);
+      sb[tid] = a.beta[(long)(base + tid) * H + h];
     }
     __syncthreads();
+    for (int t = wave; t < nt; t += 4) {               // k . q
+      float v = 0.f;
+      for (int d = lane; d < RW; d += 64) v += skq[t][d].x * skq[t][d].y;
+      v = wave_sum(v);
+      if (lane == 0) dot[t] = v;
+    }
     for (int t = 0; t < nt; ++t) {
-      float ak[V], aq[V], kq = 0.f;
-#pragma unroll
-      for (int e = 0; e < V; ++e) { ak[e] = 0.f; aq[e] = 0.f; }
-      const float* kt = sk + t * DP;
-      const float* qt = sq + t * DP;
+      f32x4 ak = {0.f, 0.f, 0.f, 0.f}, aq = ak;
+      float kr[RPT <= 16 ? RPT : 1];
 #pragma unroll
       for (int ii = 0; ii < RPT; ++ii) {
-        const int i = min(rg + RG * ii, DP - 1);       // (rows past D: S is zero there)
-        const float kv = kt[i], qv = qt[i];
-        if (rg + RG * ii < D) kq += kv * qv;
-#pragma unroll
-        for (int e = 0; e < V; ++e) { ak[e] += S[ii][e] * kv; aq[e] += S[ii][e] * qv; }
+        const float2 kq = skq[t][rg + RG * ii];
+        if constexpr (RPT <= 16) kr[ii] = kq.x;
+        ak += S[ii] * kq.x;
+        aq += S[ii] * kq.y;
       }
-      for (int o = CGP; o < 64; o <<= 1) {             // row groups inside the wave
-        kq += __shfl_xor(kq, o, 64);
 #pragma unroll
-        for (int e = 0; e < V; ++e) {
+      for (int o = CGP; o < 64; o <<= 1) {             // row groups inside the wave
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
           ak[e] += __shfl_xor(ak[e], o, 64);
           aq[e] += __shfl_xor(aq[e], o, 64);
         }
       }
-      float* pb = sp + (t & 1) * np * PW;
-      if (CGP >= 64 || lane < CGP) {
-        float* p = pb + pi * PW;
-#pragma unroll
-        for (int e = 0; e < V; ++e) {
-          p[c0 + e] = ak[e];
-          p[V * CGP + c0 + e] = aq[e];
-        }
-        if (cg == 0) p[2 * V * CGP] = kq;
+      if (lane < CGP) {
+        *reinterpret_cast<f32x4*>(&sp[t & 1][wave][0][c0]) = ak;
+        *reinterpret_cast<f32x4*>(&sp[t & 1][wave][1][c0]) = aq;
       }
       __syncthreads();
-      kq = 0.f;
+      f32x4 pk[4], pq[4];
 #pragma unroll
-      for (int e = 0; e < V; ++e) { ak[e] = 0.f; aq[e] = 0.f; }
-      for (int z = 0; z < np; ++z) {
-        const float* p = pb + z * PW;
-        kq += p[2 * V * CGP];
-#pragma unroll
-        for (int e = 0; e < V; ++e) {
-          ak[e] += p[c0 + e];
-          aq[e] += p[V * CGP + c0 + e];
-        }
+      for (int z = 0; z < 4; ++z) {
+        pk[z] = *reinterpret_cast<const f32x4*>(&sp[t & 1][z][0][c0]);
+        pq[z] = *reinterpret_cast<const f32x4*>(&sp[t & 1][z][1][c0]);
       }
-      const float at = sab[t], bt = sab[DS_TC + t];
-      float u[V];
+      const float at = sa[t];
+      const f32x4 u = (*reinterpret_cast<const f32x4*>(&sv[t][c0]) -
+                       (pk[0] + pk[1] + pk[2] + pk[3]) * at) * sb[t];
+      if (rg == 0)
+        *reinterpret_cast<f32x4*>(&so[t][c0]) = (pq[0] + pq[1] + pq[2] + pq[3]) * at + u * dot[t];
 #pragma unroll
-      for (int e = 0; e < V; ++e) {
-        u[e] = bt * (sv[t * V * CGP + c0 + e] - at * ak[e]);
-        if (rg == 0) so[t * V * CGP + c0 + e] = at * aq[e] + kq * u[e];
-      }
-#pragma unroll
-      for (int ii = 0; ii < RPT; ++ii) {
-        const float kv = rg + RG * ii < D ? kt[min(rg + RG * ii, DP - 1)] : 0.f;
-#pragma unroll
-        for (int e = 0; e < V; ++e) S[ii][e] = at * S[ii][e] + kv * u[e];
-      }
+      for (int ii = 0; ii < RPT; ++ii)
+        S[ii] = S[ii] * at + u * (RPT <= 16 ? kr[RPT <= 16 ? ii : 0] : skq[t][rg + RG * ii].x);
     }
     __syncthreads();
     for (int t = wave; t < nt; t += 4) {               // head RMS norm, weight, gate
-      const float* o = so + t * V * CGP;
       float ss = 0.f;
-      for (int d = lane; d < Dv; d += 64) ss += o[d] * o[d];
+      for (int d = lane; d < Dv; d += 64) ss += so[t][d] * so[t][d];
       const float inv = a.out_scale / sqrtf(wave_sum(ss) / (float)Dv + a.eps);
       for (int d = lane; d < Dv; d += 64)
         st_f32<T>(Y + (long)(base + t) * a.ldy, (long)h * Dv + d,
-                  o[d] * inv * ld_f32<T>(NW, d) *
+                  so[t][d] * inv * ld_f32<T>(NW, d) *
                       dl_silu(ld_f32<T>(GT + (long)(base + t) * a.ldg, (long)h * Dv + d)));
     }
   }
 #pragma unroll
   for (int ii = 0; ii < RPT; ++ii) {
     const int i = rg + RG * ii;
-    if (!col || i >= D) continue;
-    if constexpr (V == 4)
-      *reinterpret_cast<f32x4*>(Sg + (long)i * Dv + c0) = f32x4{S[ii][0], S[ii][1], S[ii][2], S[ii][3]};
-    else
-      Sg[(long)i * Dv + c0] = S[ii][0];
+    if (i >= D || c0 >= Dv) continue;
+    if (vec) {
+      *reinterpret_cast<f32x4*>(Sg + (long)i * Dv + c0) = S[ii];
+    } else {
+#pragma unroll
+      for (int e = 0; e < 4; ++e)
+        if (c0 + e < Dv) Sg[(long)i * Dv + c0 + e] = S[ii][e];
+    }
   }
 }
 
@@ -187,26 +166,17 @@ static bool delta_args_ok(const DeltaArgs& a, int nseq) {
 
 template <typename T>
 static int delta_step(const DeltaArgs& a, int nseq, hipStream_t st) {
-  const int V = a.Dv % 4 == 0 ? 4 : 1;
-  int lg = 0;
-  while ((V << lg) < a.Dv) ++lg;
-  if (lg > 8) return EIA_UNSUPPORTED;
-  const int RG = 256 >> lg, rpt = (a.D + RG - 1) / RG, CGP = 1 << lg;
-  if (rpt > 64) return EIA_UNSUPPORTED;
-  const int np = CGP >= 64 ? RG : 4;
-  const size_t lds = sizeof(float) * (DS_TC * (2 * a.DP + 2 * V * CGP) +
-                                      2 * np * (2 * V * CGP + 4) + 2 * DS_TC);
-  if (lds > 64 * 1024) return EIA_UNSUPPORTED;
+  if (a.D > 256 || a.Dv > 256) return EIA_UNSUPPORTED;
+  const int vec = a.Dv % 4 == 0 && reinterpret_cast<uintptr_t>(a.S) % 16 == 0;
   const dim3 grid(nseq, a.H);
-#define DS_GO(VV, R) \
-  hipLaunchKernelGGL((delta_scan_kernel<T, VV, R>), grid, dim3(256), lds, st, a, lg)
-#define DS_ROWS(VV)                                                                    \
-  do {                                                                                 \
-    if (rpt <= 4) DS_GO(VV, 4); else if (rpt <= 8) DS_GO(VV, 8);                       \
-    else if (rpt <= 16) DS_GO(VV, 16); else if (rpt <= 32) DS_GO(VV, 32);              \
-    else DS_GO(VV, 64);                                                                \
+#define DS_GO(LG, R) \
+  hipLaunchKernelGGL((delta_scan_kernel<T, LG, R>), grid, dim3(256), 0, st, a, vec)
+#define DS_ROWS(LG, R)                                                                \
+  do {                                                                                \
+    if (a.D <= 64) DS_GO(LG, R); else if (a.D <= 128) DS_GO(LG, 2 * R);               \
+    else DS_GO(LG, 4 * R);                                                            \
   } while (0)
-  if (V == 4) DS_ROWS(4); else DS_ROWS(1);
+  if (a.Dv <= 64) DS_ROWS(4, 4); else if (a.Dv <= 128) DS_ROWS(5, 8); else DS_ROWS(6, 16);
 #undef DS_ROWS
 #undef DS_GO
   EIA_LAUNCH_CHECK();

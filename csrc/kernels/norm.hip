@@ -613,33 +613,34 @@ EIA_API int eia_post_rms(const void* y, long ldy, const float* ypart, int sk, co
 // arrays.  NS = 1 with mix = outw = in_next = 1 is the plain residual sum.  All arithmetic fp32.
 constexpr int HC_MAX = 8;
 
-// V: columns per thread and step (4: 16-byte accesses; needs W, ldy and ldh multiples of 4)
-template <typename T, int V>
-__global__ void __launch_bounds__(256)
+// V: columns per thread and step (4: 16-byte accesses; needs W, ldy and ldh multiples of 4);
+// NM: upper bound of NS the registers are sized for
+template <typename T, int V, int NM>
+__global__ void __launch_bounds__(512)
 hyper_step_kernel(float* __restrict__ X, int NS, int W, const T* __restrict__ y, long ldy,
                   const float* __restrict__ part, int sk, long pstride,
                   const T* __restrict__ ybias, const float* __restrict__ mix,
                   const float* __restrict__ outw, float ymult, const float* __restrict__ in_next,
                   const T* __restrict__ w_next, float w_off, T* __restrict__ h, long ldh,
                   float eps) {
-  __shared__ float scratch[4];
+  __shared__ float scratch[8];
   extern __shared__ float u_s[];                    // [W] when h is given
   const long row = blockIdx.x;
   float* xr = X + row * (long)NS * W;
   const bool upd = y || part;
-  float mx[HC_MAX][HC_MAX], ow[HC_MAX], iw[HC_MAX];
+  float mx[NM][NM], ow[NM], iw[NM];
 #pragma unroll
-  for (int s = 0; s < HC_MAX; ++s) {
+  for (int s = 0; s < NM; ++s) {
     ow[s] = (upd && s < NS) ? ymult * outw[s] : 0.f;
     iw[s] = (h && s < NS) ? in_next[s] : 0.f;
 #pragma unroll
-    for (int j = 0; j < HC_MAX; ++j) mx[s][j] = (upd && s < NS && j < NS) ? mix[s * NS + j] : 0.f;
+    for (int j = 0; j < NM; ++j) mx[s][j] = (upd && s < NS && j < NS) ? mix[s * NS + j] : 0.f;
   }
   float ss = 0.f;
   for (int c = V * threadIdx.x; c < W; c += V * blockDim.x) {
-    float xs[HC_MAX][V];
+    float xs[NM][V];
 #pragma unroll
-    for (int s = 0; s < HC_MAX; ++s) {
+    for (int s = 0; s < NM; ++s) {
       if (s < NS) {
         if constexpr (V == 4) {
           const f32x4 v = *reinterpret_cast<const f32x4*>(xr + (long)s * W + c);
@@ -667,28 +668,33 @@ hyper_step_kernel(float* __restrict__ X, int NS, int W, const T* __restrict__ y,
 #pragma unroll
         for (int e = 0; e < V; ++e) yv[e] = ybias ? ld_f32<T>(ybias, c + e) : 0.f;
         const float* p = part + row * (long)W + c;
-        for (int z = 0; z < sk; ++z) {
-          if constexpr (V == 4) {
-            const f32x4 v = *reinterpret_cast<const f32x4*>(p + z * pstride);
+        if constexpr (V == 4) {
+          for (int z0 = 0; z0 < sk; z0 += 8) {         // eight partials in flight
+            f32x4 v[8];
 #pragma unroll
-            for (int e = 0; e < V; ++e) yv[e] += v[e];
-          } else {
-            yv[0] += p[z * pstride];
+            for (int z = 0; z < 8; ++z)
+              v[z] = *reinterpret_cast<const f32x4*>(p + min(z0 + z, sk - 1) * pstride);
+#pragma unroll
+            for (int z = 0; z < 8; ++z)
+#pragma unroll
+              for (int e = 0; e < V; ++e) yv[e] += z0 + z < sk ? v[z][e] : 0.f;
           }
+        } else {
+          for (int z = 0; z < sk; ++z) yv[0] += p[z * pstride];
         }
       }
-      float nx[HC_MAX][V];
+      float nx[NM][V];
 #pragma unroll
-      for (int j = 0; j < HC_MAX; ++j)
+      for (int j = 0; j < NM; ++j)
 #pragma unroll
         for (int e = 0; e < V; ++e) {
           float v = ow[j] * yv[e];
 #pragma unroll
-          for (int s = 0; s < HC_MAX; ++s) v += mx[s][j] * xs[s][e];
+          for (int s = 0; s < NM; ++s) v += mx[s][j] * xs[s][e];
           nx[j][e] = v;
         }
 #pragma unroll
-      for (int j = 0; j < HC_MAX; ++j) {
+      for (int j = 0; j < NM; ++j) {
         if (j < NS) {
           if constexpr (V == 4)
             *reinterpret_cast<f32x4*>(xr + (long)j * W + c) =
@@ -705,7 +711,7 @@ hyper_step_kernel(float* __restrict__ X, int NS, int W, const T* __restrict__ y,
       for (int e = 0; e < V; ++e) {
         float u = 0.f;
 #pragma unroll
-        for (int j = 0; j < HC_MAX; ++j) u += iw[j] * xs[j][e];
+        for (int j = 0; j < NM; ++j) u += iw[j] * xs[j][e];
         u_s[c + e] = u;
         ss += u * u;
       }
@@ -735,18 +741,25 @@ EIA_API int eia_hyper_step(float* X, int NS, int W, const void* y, long ldy, con
   if ((size_t)W * sizeof(float) > 64 * 1024) return EIA_UNSUPPORTED;
   if (rows == 0) return EIA_OK;
   const bool vec = W % 4 == 0 && ldy % 4 == 0 && ldh % 4 == 0;
-  const int threads = W >= 1024 ? 256 : (W >= 512 ? 128 : 64);
+  // (few rows: one pass over the row, so every load of a thread is in flight at once)
+  const int threads = W >= 2048 && rows <= 512 ? 512 : W >= 1024 ? 256 : (W >= 512 ? 128 : 64);
   const size_t lds = h ? sizeof(float) * W : 0;
   const long ps = (long)rows * W;
-#define HC_LAUNCH(TT, VV)                                                                        \
-  hipLaunchKernelGGL((hyper_step_kernel<TT, VV>), dim3(rows), dim3(threads), lds, st, X, NS, W,  \
+#define HC_LAUNCH1(TT, VV, NN)                                                                   \
+  hipLaunchKernelGGL((hyper_step_kernel<TT, VV, NN>), dim3(rows), dim3(threads), lds, st, X, NS, W,  \
                      (const TT*)y, ldy, part, sk, ps, (const TT*)ybias, mix, outw, ymult,        \
                      in_next, (const TT*)w_next, w_off, (TT*)h, ldh, eps)
+#define HC_LAUNCH(TT, VV)                                                                        \
+  do {                                                                                           \
+    if (NS <= 2) HC_LAUNCH1(TT, VV, 2); else if (NS <= 4) HC_LAUNCH1(TT, VV, 4);                 \
+    else HC_LAUNCH1(TT, VV, HC_MAX);                                                             \
+  } while (0)
   if (is_bf16) {
     if (vec) HC_LAUNCH(bf16_t, 4); else HC_LAUNCH(bf16_t, 1);
   } else {
     if (vec) HC_LAUNCH(float, 4); else HC_LAUNCH(float, 1);
   }
 #undef HC_LAUNCH
+#undef HC_LAUNCH1
   EIA_LAUNCH_CHECK();
 }
