@@ -66,12 +66,27 @@ def kernel_sources() -> list[str]:
     return sorted(os.path.join(kd, f) for f in os.listdir(kd) if f.endswith(".hip"))
 
 
-def build_kernels(force: bool = False, jobs: int = 8) -> str:
+def partial_so(only) -> str:
+    """Path of the library that holds the kernel sources ``only`` (file stems)."""
+    import hashlib
+    tag = hashlib.sha256("\n".join(sorted(only)).encode()).hexdigest()[:8]
+    return os.path.join(OUT_DIR, f"libeia_kernels_{tag}.so")
+
+
+def build_kernels(force: bool = False, jobs: int = 8, only=None) -> str:
+    """Compile and link the kernel library; ``only``: a library of these source files (stems)
+    alone, for a first use that needs no others (objects are shared with the whole library)."""
     if not HIPCC or not os.path.exists(HIPCC):
         raise RuntimeError("hipcc not found; ROCm toolchain required to build gfx950 kernels")
     os.makedirs(OUT_DIR, exist_ok=True)
     os.makedirs(OBJ_DIR, exist_ok=True)
     srcs = kernel_sources()
+    target = KERNELS_SO
+    if only is not None:
+        srcs = [p for p in srcs if os.path.basename(p)[:-len(".hip")] in set(only)]
+        if len(srcs) != len(set(only)):
+            raise ValueError(f"unknown kernel sources among {sorted(only)}")
+        target = partial_so(only)
     hdrs = _headers()
     objs = []
     todo = []
@@ -86,19 +101,20 @@ def build_kernels(force: bool = False, jobs: int = 8) -> str:
             f.result()
     # the link also re-runs when the source SET changed (a kernel file deleted or added):
     # the library must not keep symbols of sources that no longer exist
-    manifest = os.path.join(OBJ_DIR, "kernels.manifest")
+    manifest = os.path.join(OBJ_DIR, "kernels.manifest" if only is None else
+                            os.path.basename(target) + ".manifest")
     want = "\n".join(os.path.basename(o) for o in objs)
     try:
         have = open(manifest).read()
     except OSError:
         have = None
-    if force or todo or have != want or not _newer(KERNELS_SO, objs):
-        tmp = KERNELS_SO + ".tmp"
+    if force or todo or have != want or not _newer(target, objs):
+        tmp = target + ".tmp"
         _run([HIPCC, f"--offload-arch={ARCH}", "-shared", "-fPIC", "-o", tmp, *objs])
-        os.replace(tmp, KERNELS_SO)
+        os.replace(tmp, target)
         with open(manifest, "w") as f:
             f.write(want)
-    return KERNELS_SO
+    return target
 
 
 def build_runtime(force: bool = False) -> str:

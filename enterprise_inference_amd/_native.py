@@ -139,20 +139,32 @@ def gpu_available() -> bool:
     return torch.cuda.is_available()
 
 
-def _build_kernels() -> None:
+def _builder():
     root = os.path.dirname(os.path.dirname(_LIB_DIR))
     spec = importlib.util.spec_from_file_location("eia_build", os.path.join(root, "csrc", "build.py"))
     mod = importlib.util.module_from_spec(spec)
     spec.loader.exec_module(mod)
-    mod.build_kernels()
+    return mod
 
 
-def _build_runtime() -> None:
-    root = os.path.dirname(os.path.dirname(_LIB_DIR))
-    spec = importlib.util.spec_from_file_location("eia_build", os.path.join(root, "csrc", "build.py"))
-    mod = importlib.util.module_from_spec(spec)
-    spec.loader.exec_module(mod)
-    mod.build_runtime()
+def _bind(lib: ctypes.CDLL, names) -> None:
+    for name in names:
+        fn = getattr(lib, name)
+        fn.argtypes = _SIGNATURES[name]
+        fn.restype = ctypes.c_int
+
+
+def _load_whole() -> ctypes.CDLL:
+    if not os.path.exists(_KERNELS_SO):
+        _builder().build_kernels()
+    lib = ctypes.CDLL(_KERNELS_SO, mode=ctypes.RTLD_GLOBAL)
+    missing = [n for n in _SIGNATURES if not hasattr(lib, n)]
+    if missing:
+        # a stale build: fail here, not at the first call of the missing kernel
+        raise RuntimeError(f"{_KERNELS_SO} lacks {missing}; rebuild it "
+                           "(python -c 'import __graft_entry__ as g; g.build()')")
+    _bind(lib, _SIGNATURES)
+    return lib
 
 
 def kernels() -> ctypes.CDLL:
@@ -161,22 +173,37 @@ def kernels() -> ctypes.CDLL:
     if _kernels is not None:
         return _kernels
     with _lock:
+        if _kernels is None:
+            _kernels = _load_whole()
+        return _kernels
+
+
+def prepare(sources) -> None:
+    """Where the kernel library is not built yet, compile and load only ``sources`` (the stems of
+    csrc/kernels files a model runs on).  A kernel outside them builds and loads the whole library at
+    its first call.  Nothing happens when the library is there or ``sources`` is empty."""
+    global _kernels
+    if not sources or os.path.exists(_KERNELS_SO):
+        return
+    with _lock:
         if _kernels is not None:
-            return _kernels
-        if not os.path.exists(_KERNELS_SO):
-            _build_kernels()
-        lib = ctypes.CDLL(_KERNELS_SO, mode=ctypes.RTLD_GLOBAL)
-        missing = [n for n in _SIGNATURES if not hasattr(lib, n)]
-        if missing:
-            # a stale build: fail here, not at the first call of the missing kernel
-            raise RuntimeError(f"{_KERNELS_SO} lacks {missing}; rebuild it "
-                               "(python -c 'import __graft_entry__ as g; g.build()')")
-        for name, argtypes in _SIGNATURES.items():
-            fn = getattr(lib, name)
-            fn.argtypes = argtypes
-            fn.restype = ctypes.c_int
+            return
+        lib = ctypes.CDLL(_builder().build_kernels(only=sources))
+        have = [n for n in _SIGNATURES if hasattr(lib, n)]
+        _bind(lib, have)
+
+        def outside(name):
+            def call(*args):
+                global _kernels
+                with _lock:
+                    if _kernels is lib:
+                        _kernels = _load_whole()
+                return getattr(_kernels, name)(*args)
+            return call
+
+        for name in set(_SIGNATURES) - set(have):
+            setattr(lib, name, outside(name))
         _kernels = lib
-        return lib
 
 
 def runtime():
@@ -192,7 +219,7 @@ def runtime():
         try:
             _runtime = importlib.import_module("_eia_runtime")
         except ImportError:
-            _build_runtime()
+            _builder().build_runtime()
             importlib.invalidate_caches()
             _runtime = importlib.import_module("_eia_runtime")
         return _runtime

@@ -114,6 +114,7 @@ def main(argv=None) -> int:
     import numpy as np
     import torch
 
+    from .. import _native
     from ..config import parse_dtype
     from ..models import get_model_class
     from ..models.loader import resolve_model_config
@@ -123,10 +124,13 @@ def main(argv=None) -> int:
     if device == "auto":
         device = "cuda" if torch.cuda.is_available() else "cpu"
     mcfg = resolve_model_config(a.model)
-    if dtype == torch.float32 and device == "cuda" and not getattr(
-            get_model_class(mcfg.architecture), "supports_float32", False):
+    cls = get_model_class(mcfg.architecture)
+    if dtype == torch.float32 and device == "cuda" and not getattr(cls, "supports_float32", False):
         print(f"{mcfg.architecture} has no float32 kernels", file=sys.stderr)
         return 3
+    if device == "cuda":
+        # in a fresh checkout: compile this model's kernels only
+        _native.prepare(getattr(cls, "kernel_sources", None))
     sess = TraceSession(replay_config(mcfg, a.model, dtype, device, a.max_tokens))
     os.makedirs(a.out, exist_ok=True)
     for line in sys.stdin:

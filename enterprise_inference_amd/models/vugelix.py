@@ -93,6 +93,9 @@ def weight_owners(specs) -> list:
 
 class VugelixForCausalLM(HyperConnectedDecoder):
     supports_graphs = True         # no step reads anything back to the host
+    # csrc/kernels files of a step without sampling
+    kernel_sources = ("activation", "delta_prep", "delta_scan", "embed", "gemm_skinny", "norm",
+                      "window_attention")
 
     def __init__(self, cfg: ModelConfig, dtype=torch.bfloat16, device=None):
         super().__init__()
