@@ -274,13 +274,6 @@ def prefill_plan(md, device) -> Optional[ChunkPlan]:
     return md.work_cache["delta_chunks"]
 
 
-def chunked_pays(plan: ChunkPlan, heads: int) -> bool:
-    """Whether the chunk-parallel form beats the token-by-token one for a step's portions."""
-    if FORCE_CHUNKED is not None:
-        return FORCE_CHUNKED
-    return True
-
-
 def delta_scan(rows: DeltaRows, spec: DeltaSpec, state: DeltaState, md, norm_w: torch.Tensor,
                out: Optional[torch.Tensor] = None, plan: Optional[ChunkPlan] = None) -> torch.Tensor:
     """-> y [T, H*dv] in the gate's dtype (``out``: a view to write into).  ``norm_w`` [dv].  Updates
@@ -343,7 +336,7 @@ def delta_scan(rows: DeltaRows, spec: DeltaSpec, state: DeltaState, md, norm_w: 
 
     nseq = md.num_seqs if md.num_seqs else T
     if (plan is None or not plan.n or max(D, Dv) > CHUNK_MAX_DIM or md.seq_cu is None or
-            plan.rows != T or not chunked_pays(plan, H) or torch.cuda.is_current_stream_capturing()):
+            plan.rows != T or FORCE_CHUNKED is False or torch.cuda.is_current_stream_capturing()):
         step(0, nseq)
         return out
     nd = nseq - plan.nseq                       # decode rows stay token by token

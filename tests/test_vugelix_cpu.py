@@ -117,3 +117,20 @@ def test_random_initialisation_keeps_pads_zero():
         o, mix = L.mix.o.data, L.mix
         assert not o[:, mix.lw:mix.lw_pad].any() and not o[:, mix.lw_pad + mix.rw:].any()
         assert o[:, :mix.lw].any() and bool(torch.isfinite(mix.right.spec.exp_a).all())
+
+
+def test_kernel_source_subset_has_a_library_of_its_own():
+    import importlib.util
+    import os
+    root = os.path.dirname(os.path.dirname(os.path.abspath(__file__)))
+    spec = importlib.util.spec_from_file_location("eia_build", os.path.join(root, "csrc", "build.py"))
+    b = importlib.util.module_from_spec(spec)
+    spec.loader.exec_module(b)
+    from enterprise_inference_amd.models.vugelix import VugelixForCausalLM
+    stems = [os.path.basename(p)[:-4] for p in b.kernel_sources()]
+    src = VugelixForCausalLM.kernel_sources
+    assert set(src) < set(stems)
+    assert b.partial_so(src) == b.partial_so(tuple(reversed(src))) != b.KERNELS_SO
+    assert b.partial_so(src[:-1]) != b.partial_so(src)
+    with pytest.raises(ValueError):
+        b.build_kernels(only=("no_such_file",))

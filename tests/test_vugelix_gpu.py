@@ -105,6 +105,36 @@ def test_generate_graph_decode():
     K.case_generate("cuda", torch.bfloat16, C.config_c, expect_graphs=True)
 
 
+@pytest.mark.parametrize("dtype", DTYPES, ids=IDS)
+def test_declared_kernel_sources_cover_a_step(dtype):
+    """Every kernel that a replayed step launches comes from the source files the model declares (a
+    fresh checkout compiles those alone)."""
+    import os
+    import re
+
+    from enterprise_inference_amd import _native
+    from enterprise_inference_amd.models.vugelix import VugelixForCausalLM
+    kdir = os.path.join(os.path.dirname(os.path.dirname(os.path.abspath(__file__))), "csrc", "kernels")
+    declared = set()
+    for stem in VugelixForCausalLM.kernel_sources:
+        with open(os.path.join(kdir, stem + ".hip")) as f:
+            declared |= set(re.findall(r"EIA_API int (eia_\w+)", f.read()))
+    real, used = _native.kernels(), set()
+
+    class Recorder:
+        def __getattr__(self, name):
+            used.add(name)
+            return getattr(real, name)
+
+    _native._kernels = Recorder()
+    try:
+        for cfg in (C.config_a, C.config_c):
+            K.case_schedules("cuda", dtype, cfg, seed=7, block_size=32)
+    finally:
+        _native._kernels = real
+    assert "eia_delta_prep" in used and used <= declared, used - declared
+
+
 def test_native_library_loaded():
     from enterprise_inference_amd import _native
     lib = _native.kernels()
